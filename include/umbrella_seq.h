@@ -4,7 +4,7 @@
  * libumbrella_hip.so: gated linear attention (a per-head matrix state carried from token to token) and sliding-window
  * attention over a paged key/value store with mean-pooled blocks behind the window and sigmoid (un-normalised) weights;
  * latent attention; a minimal gated recurrence; softmax attention with a bias by distance beside a state-space layer with a
- * scalar decay per head; residuals of one or several streams; dense, PolyNorm and routed-expert feed-forwards.
+ * scalar decay per head; differential attention over chunks of positions; attention with a sink beside a gated delta rule; residuals of one or several streams; dense, PolyNorm and routed-expert feed-forwards.
  * The layer list, every size and every constant are data (UmbSeqLayer); one forward entry point walks the list.
  *
  * Conventions are those of umbrella_hip.h: extern "C", plain pointers and sizes, 0 or a negative errno-style code,
@@ -29,7 +29,7 @@ typedef struct ihipStream_t* umb_stream_t;   /* == hipStream_t */
 
 enum { UMB_SEQ_F16 = 0, UMB_SEQ_BF16 = 1, UMB_SEQ_F32 = 2 };
 enum { UMB_MIX_POOLED_WINDOW = 0, UMB_MIX_GLA = 1, UMB_MIX_LATENT = 2, UMB_MIX_MINGRU = 3, UMB_MIX_ATTN_SSD = 4,
-       UMB_MIX_RETENTION = 5, UMB_MIX_ATTN_MLSTM = 6 };
+       UMB_MIX_RETENTION = 5, UMB_MIX_ATTN_MLSTM = 6, UMB_MIX_DIFF_ATTN = 7, UMB_MIX_ATTN_DELTA = 8 };
 /* feed-forward kinds: gated SiLU (W_down (silu(W_gate h) * W_up h)), PolyNorm (W_down polynorm(W_up h)), routed experts */
 enum { UMB_FF_GATED = 0, UMB_FF_POLYNORM = 1, UMB_FF_MOE = 2 };
 /* activation of a feed-forward / expert: silu(W_gate h) * (W_up h) over stacked [gate; up], relu(W_up h)^2 (no gate), or the
@@ -72,12 +72,17 @@ int umb_seq_linear_grouped(void* out, const void* x, const void* w, const int* t
  * x fp32 [*][W]; rows: optional gather (row i of out comes from row rows[i] of x); out_f32 and/or out_dt may be given. */
 int umb_seq_group_norm(float* out_f32, void* out_dt, const float* x, const int* rows, const void* w, int T, int W, int groups,
                        float eps, int dtype, umb_stream_t stream);
-/* x[t] <- embed[tokens[t]] (fp32); h[t] <- group_norm(x[t]) * w in `dtype` */
-int umb_seq_embed_norm(float* x, void* h, const void* embed, const int* tokens, const void* w, int T, int W, int V, int groups,
-                       float eps, int dtype, umb_stream_t stream);
+/* x[t] <- embed[tokens[t]] * scale (fp32); h[t] <- group_norm(x[t]) * w in `dtype` */
+int umb_seq_embed_norm(float* x, void* h, const void* embed, const int* tokens, float scale, const void* w, int T, int W, int V,
+                       int groups, float eps, int dtype, umb_stream_t stream);
 /* x <- x + group_norm(y) * w_post ; if w_next: h <- group_norm(x) * w_next in `dtype`   (y fp32 [T][W]) */
 int umb_seq_resid_norm(float* x, void* h, const float* y, const void* w_post, const void* w_next, int T, int W, int groups,
                        float eps, int dtype, umb_stream_t stream);
+
+/* m = coef (norm(y1) * w1 + norm(y2) * w2); x <- x + norm(m) * w_post; if w_next: h <- norm(x) * w_next in `dtype` (plain RMS
+ * norms over the row; y1, y2 fp32 [T][W]): the seam behind two mixers side by side */
+int umb_seq_pair_resid_norm(float* x, void* h, const float* y1, const float* y2, const void* w1, const void* w2, float coef,
+                            const void* w_post, const void* w_next, int T, int W, float eps, int dtype, umb_stream_t stream);
 
 /* x[t] <- embed[tokens[t]] * scale (fp32) */
 int umb_seq_embed(float* x, const void* embed, const int* tokens, float scale, int T, int W, int V, int dtype,
@@ -276,6 +281,48 @@ int umb_bsa_attend_tiled(void* out, int ldo, const float* q, const UmbPagedKV* k
                          const int* seq_len, int B, int max_len, int H, int G, int D, int E, int window, float scale,
                          float out_scale, float softcap, int dtype, umb_stream_t stream);
 
+/* ---- the same attention in its general form.  UmbAttnForm: maps 2: differential attention (every head has two query / key maps
+ * over the same values: q [T][H][2][D], cached key rows [map 1 | map 2] of 2 D; a head's output is a1 - lambda a2 over its root
+ * mean square (eps), times out_scale and the gate); chunk > 0: position i sees only keys of its own run of `chunk` positions
+ * counted from position 0; sink fp32 [H] (null: none): exp(sink[h]) joins the softmax denominator.
+ * prep: columns [q (H maps D) | k (G maps D) | v (G E)] of proj, with append 0 [q] alone (the keys and values are another layer's);
+ * norm_qk / norm_v: unit RMS per head (and map), w_q / w_k [D] null: 1; then rotary positions on the first rot_dims features of
+ * every map (layout 0: i with i + rot_dims / 2, 1: 2i with 2i + 1; cos and sin times rot_mult); query temperature as above.
+ * umb_bsa_prep / umb_bsa_attend / umb_bsa_attend_tiled are the cases without a form. */
+typedef struct UmbAttnForm { int32_t maps, chunk; const float* sink; float lambda, eps; } UmbAttnForm;
+int umb_attn_prep(float* q, const UmbPagedKV* kv, const float* proj, int ld, int append, const void* w_q, const void* w_k, int norm_qk,
+                  int norm_v, const int* pos, const int* slot, const float* freq, int rot_dims, int layout, float rot_mult, int T,
+                  int H, int G, int D, int E, int maps, float temp_coef, int temp_every, float eps, int dtype, umb_stream_t stream);
+int umb_attn_attend(void* out, int ldo, const float* q, const UmbPagedKV* kv, const float* proj, int ld, int gate_col,
+                    const float* bias, int n_dist, const int* pos, const int* slot, int T, int H, int G, int D, int E, int window,
+                    float scale, float out_scale, float softcap, const UmbAttnForm* form, float* scratch, long scratch_floats,
+                    int dtype, umb_stream_t stream);
+int umb_attn_attend_tiled(void* out, int ldo, const float* q, const UmbPagedKV* kv, const float* proj, int ld, int gate_col,
+                          const float* bias, int n_dist, const int* seq_slot, const int* seq_row0, const int* seq_pos0,
+                          const int* seq_len, int B, int max_len, int H, int G, int D, int E, int window, float scale,
+                          float out_scale, float softcap, const UmbAttnForm* form, int dtype, umb_stream_t stream);
+
+/* ---- gated delta rule: per (sequence, value head) a [D][E] fp32 state, S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q.
+ * Columns of proj from col0: [q (Hk D) | k (Hk D) | v (H E) | gate (H E) | b (H) | a (H)]; q, k and v pass a causal convolution per
+ * channel (conv_w [2 Hk D + H E][taps] in `dtype`) and silu, q and k become unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q
+ * times D^-1/2; head h uses q / k head h / (H / Hk); beta = sigmoid(b), log g = -exp(a_log) softplus(a + dt_bias) (fp32 [H] each).
+ * ring fp32 [slots][taps][2 Hk D + H E]: the raw input of position p in row p % taps (D <= 256).
+ * step: steps of one token per sequence, everything above in one launch, the ring included.  prep: q, k -> [T][ldqk] in groups of
+ * D rounded up to 16 (zero padded), v [T][H E], beta and log g [T][H]; the ring is refreshed afterwards (umb_ssd_conv_update with
+ * taps + 1).  scan: the recurrence over prepared rows in chunks of 64 tokens; scratch at least umb_delta_scan_floats(..) floats (0:
+ * the shape is not covered; no stream argument), 16-byte aligned like q and k.  o fp32 [T][H E]; state fp32 [slots][H][D][E]; a
+ * sequence that starts at position 0 starts from S = 0 whatever its slot holds. */
+int umb_delta_step(float* o, float* state, const float* proj, int ld, int col0, const void* conv_w, float* ring,
+                   const float* dt_bias, const float* a_log, const int* pos, const int* slot, int T, int Hk, int H, int D, int E,
+                   int taps, int dtype, umb_stream_t stream);
+int umb_delta_prep(float* q, float* k, int ldqk, float* v, float* beta, float* log_g, const float* proj, int ld, int col0,
+                   const void* conv_w, float* ring, const float* dt_bias, const float* a_log, const int* pos, const int* slot, int T,
+                   int Hk, int H, int D, int E, int taps, int dtype, umb_stream_t stream);
+long umb_delta_scan_floats(int T, int H, int D, int E);
+int umb_delta_scan(float* o, float* state, const float* q, const float* k, int ldqk, const float* v, const float* beta,
+                   const float* log_g, const int* seq_slot, const int* seq_row0, const int* seq_pos0, const int* seq_len, int T, int B,
+                   int max_len, int Hk, int H, int D, int E, float* scratch, long scratch_floats, umb_stream_t stream);
+
 /* ---- routed experts, softmax form: scores = softmax(logits) over all experts; the `top` largest of score + correction
  * (correction fp32 [E], null: none; ties: the lower index) are chosen; wt = the chosen scores over (their sum + 1e-20). */
 int umb_moe_route_softmax(int* sel, float* wt, const float* logits, const float* correction, int T, int E, int top,
@@ -428,6 +475,18 @@ typedef struct UmbSeqLayer {
   int32_t shared_gate;
   /* the embedding row is added to x once more right before this layer (a span of layers that runs again) */
   int32_t add_embed, pad4_;
+  /* differential attention (kind 7): proj = [q (heads 2 dim) | k (kv_heads 2 dim) | v (kv_heads vdim)], or [q] alone with kv_shared
+   * (kv is then another layer's store); chunk (0: none), rotary as above with rot_mult on cos and sin, diff_lambda, out_mult.
+   * attention with a sink beside a gated delta rule (kind 8), both reading the same input: proj = [q | k | v | dq | dk | dv | gate | b | a];
+   * attention: heads / kv_heads / dim / vdim / scale, q_norm / k_norm [dim], attn_sink fp32 [heads]; delta rule: s_heads value heads x
+   * s_vdim over s_groups q / k heads x s_state, s_taps taps (s_conv, s_conv_state [slots][s_taps][channels]), s_a_log, s_dt_bias, s_norm
+   * [s_vdim], state; each has its own output projection (out, out2), and pair_coef (norm(.) out_norm_a + norm(.) out_norm_b) of
+   * the two is the mixer's output (norms plain, over the width) */
+  int32_t chunk, kv_shared;
+  float rot_mult, diff_lambda, out_mult, pair_coef;
+  const float* attn_sink;
+  UmbSeqLinear out2;
+  const void *out_norm_a, *out_norm_b;
 } UmbSeqLayer;
 
 typedef struct UmbSeqModel {
@@ -466,7 +525,7 @@ typedef struct UmbSeqWork {
   int64_t moe_max_tiles;
   int64_t aux_floats;  /* floats in aux (what a step does not use of it serves as scratch) */
   void* h2;            /* parallel blocks: normed input of the feed-forward [Tmax][W] dtype */
-  float* y2;           /* parallel blocks: feed-forward output [Tmax][W] fp32 */
+  float* y2;           /* parallel blocks: feed-forward output; mixers with two output projections: the second [Tmax][W] fp32 */
 } UmbSeqWork;
 
 typedef struct UmbSeqStep {

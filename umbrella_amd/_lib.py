@@ -241,7 +241,14 @@ class UmbSeqLayer(C.Structure):
                 ("m_heads", C.c_int32), ("m_dim", C.c_int32), ("m_vdim", C.c_int32), ("m_pad", C.c_int32),
                 ("m_norm", C.c_void_p), ("m_max", C.c_void_p),
                 ("act_limit", C.c_float), ("shared_limit", C.c_float), ("act_alpha", C.c_float), ("shared_gate", C.c_int32),
-                ("add_embed", C.c_int32), ("pad4_", C.c_int32)]
+                ("add_embed", C.c_int32), ("pad4_", C.c_int32),
+                ("chunk", C.c_int32), ("kv_shared", C.c_int32), ("rot_mult", C.c_float), ("diff_lambda", C.c_float),
+                ("out_mult", C.c_float), ("pair_coef", C.c_float), ("attn_sink", C.c_void_p), ("out2", UmbSeqLinear),
+                ("out_norm_a", C.c_void_p), ("out_norm_b", C.c_void_p)]
+
+
+class UmbAttnForm(C.Structure):
+    _fields_ = [("maps", C.c_int32), ("chunk", C.c_int32), ("sink", C.c_void_p), ("lambda_", C.c_float), ("eps", C.c_float)]
 
 
 class UmbSeqModel(C.Structure):
@@ -269,6 +276,7 @@ class UmbSeqStep(C.Structure):
 
 
 _PKV = C.POINTER(UmbPagedKV)
+_FORM = C.POINTER(UmbAttnForm)
 SEQ_SIGNATURES = {
     "umb_seq_linear": [_P, _P, _P, _P, _I, _I, _I, _I, _I],
     "umb_seq_linear_batched": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _L, _L, _L, _I, _P, _I, _I, _I],
@@ -290,7 +298,7 @@ SEQ_SIGNATURES = {
     "umb_lat_attend_tiled": [_P, _P, _PKV, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I],
     "umb_lat_attend_tiled_ok": [_I, _I, _I, _I],
     "umb_seq_group_norm": [_P, _P, _P, _P, _P, _I, _I, _I, _F, _I],
-    "umb_seq_embed_norm": [_P, _P, _P, _P, _P, _I, _I, _I, _I, _F, _I],
+    "umb_seq_embed_norm": [_P, _P, _P, _P, _F, _P, _I, _I, _I, _I, _F, _I],
     "umb_seq_resid_norm": [_P, _P, _P, _P, _P, _I, _I, _I, _F, _I],
     "umb_gla_decay": [_P, _P, _I, _I, _P, _P, _I, _I, _I, _F, _I],
     "umb_gla_scan": [_P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _F],
@@ -313,6 +321,14 @@ SEQ_SIGNATURES = {
     "umb_bsa_prep": [_P, _PKV, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _I],
     "umb_bsa_attend": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _L, _I],
     "umb_bsa_attend_tiled": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I],
+    "umb_attn_prep": [_P, _PKV, _P, _I, _I, _P, _P, _I, _I, _P, _P, _P, _I, _I, _F, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I],
+    "umb_attn_attend": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _FORM, _P, _L, _I],
+    "umb_attn_attend_tiled": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _FORM, _I],
+    "umb_seq_pair_resid_norm": [_P, _P, _P, _P, _P, _P, _F, _P, _P, _I, _I, _F, _I],
+    "umb_delta_step": [_P, _P, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I],
+    "umb_delta_prep": [_P, _P, _I, _P, _P, _P, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I],
+    "umb_delta_scan_floats": [_I, _I, _I, _I],
+    "umb_delta_scan": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _L],
     "umb_seq_linear_glu": [_P, _P, _P, _P, _I, _I, _I, _F, _F, _I],
     "umb_seq_linear_grouped_glu": [_P, _P, _P, _P, _I, _I, _L, _I, _I, _F, _F, _I],
     "umb_blk_seam": [_P, _P, _P, _P, _P, _P, _P, _I, _F, _P, _P, _F, _I, _I, _I, _F, _I],
@@ -335,7 +351,7 @@ SEQ_SIGNATURES = {
     "umb_seq_version": [],
 }
 _SEQ_NO_STREAM = {"umb_lat_attend_tiled_ok", "umb_seq_resid_canon_step_ok", "umb_bsa_attend_tiled_ok", "umb_mingru_scratch_floats",
-                  "umb_ssd_scan_chunked_floats"}          # predicates: no stream argument, the value is the answer
+                  "umb_ssd_scan_chunked_floats", "umb_delta_scan_floats"}          # predicates: no stream argument, the value is the answer
 _seq_lib = None
 
 

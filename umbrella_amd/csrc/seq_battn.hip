@@ -7,6 +7,15 @@
 // clamped distance itself (whatever bucketing a design uses is expanded into it at load).  Keys and values are cached as
 // normed (storage dtype); queries, scores, weights, maxima and sums are fp32 (expf, not the fast intrinsic).
 //
+// The general form (umb_attn_*, UmbAttnForm) adds, each by parameter:
+//   chunk   position i sees only keys of its own run of `chunk` positions, counted from position 0 of the sequence
+//   sink    a per-head score that joins the softmax denominator with no key and no value
+//   maps    2: differential attention -- every head has two query / key maps over the SAME values (a cached key row is [map 1 |
+//           map 2]); with a1, a2 their softmax outputs o = a1 - lambda a2, and the head's o over its root mean square goes out.
+//           The two maps of a head are two rows of one workgroup: the value rows are read once for both.
+// and its prep adds rotary positions (either pair layout, a constant on cos and sin), norms by choice, and queries alone (a
+// layer that reads another layer's keys and values).
+//
 // prep: one wave per (token, head slot): query heads -> fp32 q, key heads -> cache K, value heads -> cache V.
 // attend (vector pipe, any dtype and head size): workgroup = (token, RH query heads of ONE key/value head, so one pass over
 // the keys serves them all); waves take 64-key rounds by round number; score phase lane = key, value phase lane = value
@@ -16,48 +25,84 @@
 
 static inline bool bsa_kv_ok(const UmbPagedKV* kv) { return kv && kv->k && kv->v && kv->pages && kv->page >= 1 && kv->max_pages >= 1; }
 
+// HQ = H maps query slots, GK = G maps key slots (key slot x: key/value head x / maps, map x % maps), G value slots (GV = 0: none)
+struct AttnPrep {
+  int HQ, GK, G, GV, D, E, maps;
+  int norm_qk, norm_v;                     // unit RMS (times the weight, where there is one) of q and k; of v
+  int rot_dims, layout;
+  float rot_mult;
+  float temp_coef;
+  int temp_every;
+  float eps;
+};
+
 template <typename P>
-__global__ __launch_bounds__(256) void bsa_prep_kernel(float* __restrict__ q, UmbPagedKV kv, const float* __restrict__ proj, int ld,
-                                                       const typename El<P>::type* __restrict__ w_q,
-                                                       const typename El<P>::type* __restrict__ w_k, const int* __restrict__ pos,
-                                                       const int* __restrict__ slot, int T, int H, int G, int D, int E,
-                                                       float temp_coef, int temp_every, float eps) {
+__global__ __launch_bounds__(256) void attn_prep_kernel(float* __restrict__ q, UmbPagedKV kv, const float* __restrict__ proj, int ld,
+                                                        const typename El<P>::type* __restrict__ w_q,
+                                                        const typename El<P>::type* __restrict__ w_k, const int* __restrict__ pos,
+                                                        const int* __restrict__ slot, const float* __restrict__ freq, int T,
+                                                        AttnPrep a) {
   typedef typename El<P>::type El_;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int per = H + 2 * G;
+  const int per = a.HQ + a.GK + a.GV;
   const long item = (long)blockIdx.x * 4 + wave;
   if (item >= (long)T * per) return;
   const int t = (int)(item / per), hs = (int)(item % per);
-  const int n = hs < H + G ? D : E;
-  const int col = hs < H ? hs * D : (hs < H + G ? H * D + (hs - H) * D : H * D + G * D + (hs - H - G) * E);
+  const bool is_v = hs >= a.HQ + a.GK, is_q = hs < a.HQ;
+  const int n = is_v ? a.E : a.D, D = a.D;
+  const int col = is_v ? (a.HQ + a.GK) * D + (hs - a.HQ - a.GK) * a.E : hs * D;
   const float* src = proj + (long)t * ld + col;
-  float ss = 0.f;
-  for (int i = lane; i < n; i += 64) { const float v = src[i]; ss += v * v; }
-  ss = wave_sum(ss);
-  const float f = 1.f / sqrtf(ss / (float)n + eps);
+  float f = 1.f;
+  if (is_v ? a.norm_v : a.norm_qk) {
+    float ss = 0.f;
+    for (int i = lane; i < n; i += 64) { const float v = src[i]; ss += v * v; }
+    ss = wave_sum(ss);
+    f = 1.f / sqrtf(ss / (float)n + a.eps);
+  }
   const int p = pos[t];
-  if (hs < H) {
-    const float temp = temp_every > 0 ? 1.f + temp_coef * logf((float)((p + 1) / temp_every + 1)) : 1.f;
-    for (int i = lane; i < n; i += 64) q[(long)t * H * D + (long)hs * D + i] = src[i] * f * (w_q ? ldf<P>(w_q + i) : 1.f) * temp;
-  } else if (hs < H + G) {
-    El_* row = reinterpret_cast<El_*>(kv.k) + pkv_tok(kv, slot[t], p, hs - H, G, D);
-    for (int i = lane; i < n; i += 64) stf<P>(row + i, src[i] * f * (w_k ? ldf<P>(w_k + i) : 1.f));
-  } else {
-    El_* row = reinterpret_cast<El_*>(kv.v) + pkv_tok(kv, slot[t], p, hs - H - G, G, E);
+  if (is_v) {
+    El_* row = reinterpret_cast<El_*>(kv.v) + pkv_tok(kv, slot[t], p, hs - a.HQ - a.GK, a.G, a.E);
     for (int i = lane; i < n; i += 64) stf<P>(row + i, src[i] * f);
+    return;
+  }
+  const El_* w = is_q ? w_q : w_k;
+  const float temp = is_q && a.temp_every > 0 ? 1.f + a.temp_coef * logf((float)((p + 1) / a.temp_every + 1)) : 1.f;
+  const int ks = hs - a.HQ;
+  El_* krow = is_q ? nullptr : reinterpret_cast<El_*>(kv.k) + pkv_tok(kv, slot[t], p, ks / a.maps, a.G, a.maps * D) + (ks % a.maps) * D;
+  float* qrow = q + ((long)t * a.HQ + (is_q ? hs : 0)) * D;
+  const int half = a.rot_dims >> 1;
+  for (int i = lane; i < n; i += 64) {
+    float v = src[i] * f * (w ? ldf<P>(w + i) : 1.f);
+    if (i < a.rot_dims) {
+      int fi, other;
+      bool first;
+      if (a.layout == 0) { first = i < half; fi = first ? i : i - half; other = first ? i + half : i - half; }
+      else { first = (i & 1) == 0; fi = i >> 1; other = i ^ 1; }
+      const float u = src[other] * f * (w ? ldf<P>(w + other) : 1.f);
+      float sn, cs;
+      sincosf((float)p * freq[fi], &sn, &cs);
+      sn *= a.rot_mult;
+      cs *= a.rot_mult;
+      v = first ? v * cs - u * sn : v * cs + u * sn;
+    }
+    if (is_q) qrow[i] = v * temp;
+    else stf<P>(krow + i, v);
   }
 }
 
 constexpr int BSA_MAXC = 8;      // value columns per lane: E <= 512
 
-template <typename P, int RH, int NC, int NW>
+// RH rows of the workgroup = RH / MAPS query heads with MAPS maps each (row r: head r / MAPS, map r % MAPS)
+template <typename P, int RH, int NC, int NW, int MAPS>
 __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::type* __restrict__ out, int ldo,
                                                              const float* __restrict__ q, UmbPagedKV kv,
                                                              const float* __restrict__ proj, int ld, int gate_col,
                                                              const float* __restrict__ bias, int n_dist,
                                                              const int* __restrict__ pos, const int* __restrict__ slot_, int H,
                                                              int G, int D, int E, int window, float scale, float out_scale,
-                                                             float softcap, float* __restrict__ part, int nsplit) {
+                                                             float softcap, UmbAttnForm form, float* __restrict__ part,
+                                                             int nsplit) {
+  static_assert(RH % MAPS == 0, "rows are whole heads");
   typedef typename El<P>::type El_;
   extern __shared__ float lds[];
   constexpr int KB = 8;
@@ -70,14 +115,16 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
   float* w_s = ml_s + NW * 2 * RH + wave * (RH * 64 + 128);
   long* off_s = reinterpret_cast<long*>(w_s + RH * 64);
   const int t = blockIdx.x, hpg = H / G;
-  const int h0 = blockIdx.y * RH, g = h0 / hpg;           // RH divides H / G: the block's heads share key/value head g
+  constexpr int RR = RH / MAPS;
+  const int h0 = blockIdx.y * RR, g = h0 / hpg;           // RR divides H / G: the block's heads share key/value head g
   const int i = pos[t], slot = slot_[t];
   for (int x = threadIdx.x; x < RH * D; x += NW * 64) {
     const int r = x / D, d = x % D;
-    q_s[r * Dp + d] = q[((long)t * H + h0 + r) * D + d];
+    q_s[r * Dp + d] = q[(((long)t * H + h0) * MAPS + r) * D + d];
   }
   __syncthreads();
-  const int j_lo = i - window + 1 > 0 ? i - window + 1 : 0;
+  int j_lo = i - window + 1 > 0 ? i - window + 1 : 0;
+  if (form.chunk > 0) j_lo = max(j_lo, i / form.chunk * form.chunk);
   const int n_keys = i - j_lo + 1;
   const bool vec = (D & 7) == 0 && sizeof(El_) == 2;
   float acc[RH][NC], m_run[RH], l_run[RH];
@@ -101,15 +148,17 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
     if (kx < n_keys) {
       const int j = j_lo + kx;
       dist = i - j;
-      const El_* kr = reinterpret_cast<const El_*>(kv.k) + pkv_tok(kv, slot, j, g, G, D);
+      const El_* kr = reinterpret_cast<const El_*>(kv.k) + pkv_tok(kv, slot, j, g, G, MAPS * D);
       off = pkv_tok(kv, slot, j, g, G, E);
       bool done = false;
       if constexpr (sizeof(El_) == 2) {
         if (vec) {
+#pragma unroll
+          for (int mp = 0; mp < MAPS; ++mp)
           for (int d = 0; d < D; d += 64) {              // eight 16-byte loads in flight, then their 64 x RH products
             u32x4 kk[8];
 #pragma unroll
-            for (int u = 0; u < 8; ++u) kk[u] = *reinterpret_cast<const u32x4*>(kr + (d + 8 * u < D ? d + 8 * u : 0));
+            for (int u = 0; u < 8; ++u) kk[u] = *reinterpret_cast<const u32x4*>(kr + mp * D + (d + 8 * u < D ? d + 8 * u : 0));
 #pragma unroll
             for (int u = 0; u < 8; ++u) {
               if (d + 8 * u >= D) break;
@@ -118,7 +167,7 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
                 const float k0 = lo_f<P>(kk[u][e]), k1 = hi_f<P>(kk[u][e]);
                 const int dd = d + 8 * u + 2 * e;
 #pragma unroll
-                for (int r = 0; r < RH; ++r) s[r] += q_s[r * Dp + dd] * k0 + q_s[r * Dp + dd + 1] * k1;
+                for (int r = mp; r < RH; r += MAPS) s[r] += q_s[r * Dp + dd] * k0 + q_s[r * Dp + dd + 1] * k1;
               }
             }
           }
@@ -126,11 +175,13 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
         }
       }
       if (!done) {
-        for (int d = 0; d < D; ++d) {
-          const float kd = ldf<P>(kr + d);
 #pragma unroll
-          for (int r = 0; r < RH; ++r) s[r] += q_s[r * Dp + d] * kd;
-        }
+        for (int mp = 0; mp < MAPS; ++mp)
+          for (int d = 0; d < D; ++d) {
+            const float kd = ldf<P>(kr + mp * D + d);
+#pragma unroll
+            for (int r = mp; r < RH; r += MAPS) s[r] += q_s[r * Dp + d] * kd;
+          }
       }
     }
     const int bi = dist < n_dist ? dist : n_dist - 1;
@@ -138,7 +189,7 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
     for (int r = 0; r < RH; ++r) {
       float sc = s[r] * scale;
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);          // capped score; the bias (if any) is added to the capped value
-      const float sv = kx < n_keys ? sc + (bias ? bias[(long)(h0 + r) * n_dist + bi] : 0.f) : -INFINITY;
+      const float sv = kx < n_keys ? sc + (bias ? bias[(long)(h0 + r / MAPS) * n_dist + bi] : 0.f) : -INFINITY;
       const float m_new = fmaxf(m_run[r], wave_max(sv));          // finite: every round has at least one key
       const float fac = expf(m_run[r] - m_new);                   // 0 on the first round (m_run = -inf)
       const float pw = kx < n_keys ? expf(sv - m_new) : 0.f;
@@ -184,12 +235,13 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
     if (lane == 0) { ml_s[(wave * RH + r) * 2] = m_run[r]; ml_s[(wave * RH + r) * 2 + 1] = l_run[r]; }
   }
   __syncthreads();
-  for (int x = threadIdx.x; x < RH * E; x += NW * 64) {
-    const int r = x / E, d = x % E;
-    float M = -INFINITY;
+  // row r of the waves' partials merged in wave order: unnormalised output of column d, maximum and denominator
+  auto merged = [&](int r, int d, float& M, float& L) -> float {
+    M = -INFINITY;
 #pragma unroll
     for (int w = 0; w < NW; ++w) M = fmaxf(M, ml_s[(w * RH + r) * 2]);
-    float o = 0.f, L = 0.f;
+    float o = 0.f;
+    L = 0.f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) {
       const float mw = ml_s[(w * RH + r) * 2];
@@ -197,60 +249,215 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
       o += lds[(w * RH + r) * Ep + d] * f;
       L += ml_s[(w * RH + r) * 2 + 1] * f;
     }
-    if (nsplit > 1) {                                  // partial result of this split: [t][h][split][E + 2] = o.., M, L
-      float* pr = part + (((long)t * H + h0 + r) * nsplit + split) * (E + 2);
-      pr[d] = o;
-      if (d == 0) { pr[E] = M; pr[E + 1] = L; }
-      continue;
+    return o;
+  };
+  auto gate_of = [&](int h) { return gate_col >= 0 ? 1.f / (1.f + expf(-proj[(long)t * ld + gate_col + h])) : 1.f; };
+  if (MAPS == 1 || nsplit > 1) {
+    for (int x = threadIdx.x; x < RH * E; x += NW * 64) {
+      const int r = x / E, d = x % E;
+      float M, L;
+      const float o = merged(r, d, M, L);
+      if (nsplit > 1) {                                // partial result of this split: [t][row][split][E + 2] = o.., M, L
+        float* pr = part + ((((long)t * H + h0) * MAPS + r) * nsplit + split) * (E + 2);
+        pr[d] = o;
+        if (d == 0) { pr[E] = M; pr[E + 1] = L; }
+        continue;
+      }
+      if (form.sink) L += expf(form.sink[h0 + r] - M);
+      stf<P>(out + (long)t * ldo + (long)(h0 + r) * E + d, out_scale * gate_of(h0 + r) * (o / L));
     }
-    const float gt = gate_col >= 0 ? 1.f / (1.f + expf(-proj[(long)t * ld + gate_col + h0 + r])) : 1.f;
-    stf<P>(out + (long)t * ldo + (long)(h0 + r) * E + d, out_scale * gt * (o / L));
+  } else {
+    // a wave per head: o = a1 - lambda a2 over its root mean square
+    for (int rr = wave; rr < RR; rr += NW) {
+      float v[NC], ss = 0.f;
+#pragma unroll
+      for (int c = 0; c < NC; ++c) {
+        const int d = dcl[c];
+        float M, L1, L2;
+        float o = merged(MAPS * rr, d, M, L1);
+        if (form.sink) L1 += expf(form.sink[h0 + rr] - M);
+        const float a2 = merged(MAPS * rr + MAPS - 1, d, M, L2);
+        if (form.sink) L2 += expf(form.sink[h0 + rr] - M);
+        o = o / L1 - form.lambda * (a2 / L2);
+        v[c] = o;
+        if (lane + 64 * c < E) ss += o * o;
+      }
+      ss = wave_sum(ss);
+      const float f = out_scale * gate_of(h0 + rr) / sqrtf(ss / (float)E + form.eps);
+#pragma unroll
+      for (int c = 0; c < NC; ++c)
+        if (lane + 64 * c < E) stf<P>(out + (long)t * ldo + (long)(h0 + rr) * E + lane + 64 * c, v[c] * f);
+    }
   }
 }
 
 // the splits of one (token, head) merged: lane s holds split s's maximum and denominator (a split that had no key carries
 // M = -inf, L = 0), the factors go round by shuffles, every sum runs over the splits in order
-template <typename P>
+template <typename P, int MAPS>
 __global__ __launch_bounds__(64) void bsa_merge_kernel(typename El<P>::type* __restrict__ out, int ldo, const float* __restrict__ part,
                                                        const float* __restrict__ proj, int ld, int gate_col, int H, int E,
-                                                       int nsplit, float out_scale) {
+                                                       int nsplit, float out_scale, UmbAttnForm form) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
-  const float* pr = part + ((long)t * H + h) * nsplit * (E + 2);
-  const float ms = lane < nsplit ? pr[lane * (E + 2) + E] : -INFINITY;
-  const float ls = lane < nsplit ? pr[lane * (E + 2) + E + 1] : 0.f;
   const float gt = gate_col >= 0 ? 1.f / (1.f + expf(-proj[(long)t * ld + gate_col + h])) : 1.f;
-  const float M = wave_max(ms);
-  const float fs = ms == -INFINITY ? 0.f : expf(ms - M);
-  float L = 0.f, f[16];
+  const float* pr[MAPS];
+  float f[MAPS][16], inv[MAPS];
 #pragma unroll
-  for (int s = 0; s < 16; ++s) {
-    f[s] = __shfl(fs, s, 64);
-    L += __shfl(ls * fs, s, 64);
+  for (int mp = 0; mp < MAPS; ++mp) {
+    pr[mp] = part + (((long)t * H + h) * MAPS + mp) * nsplit * (E + 2);
+    const float ms = lane < nsplit ? pr[mp][lane * (E + 2) + E] : -INFINITY;
+    const float ls = lane < nsplit ? pr[mp][lane * (E + 2) + E + 1] : 0.f;
+    const float M = wave_max(ms);
+    const float fs = ms == -INFINITY ? 0.f : expf(ms - M);
+    float L = 0.f;
+#pragma unroll
+    for (int s = 0; s < 16; ++s) {
+      f[mp][s] = __shfl(fs, s, 64);
+      L += __shfl(ls * fs, s, 64);
+    }
+    if (form.sink) L += expf(form.sink[h] - M);
+    inv[mp] = 1.f / L;
   }
-  const float c = out_scale * gt / L;
-  for (int d = lane; d < E; d += 64) {
+  auto column = [&](int mp, int d) -> float {
     float v[16];
 #pragma unroll
-    for (int s = 0; s < 16; ++s) v[s] = pr[(s < nsplit ? s : nsplit - 1) * (E + 2) + d];
+    for (int s = 0; s < 16; ++s) v[s] = pr[mp][(s < nsplit ? s : nsplit - 1) * (E + 2) + d];
     float o = 0.f;
 #pragma unroll
-    for (int s = 0; s < 16; ++s) o += s < nsplit ? v[s] * f[s] : 0.f;
-    stf<P>(out + (long)t * ldo + (long)h * E + d, o * c);
+    for (int s = 0; s < 16; ++s) o += s < nsplit ? v[s] * f[mp][s] : 0.f;
+    return o * inv[mp];
+  };
+  typename El<P>::type* orow = out + (long)t * ldo + (long)h * E;
+  if constexpr (MAPS == 1) {
+    const float c = out_scale * gt;
+    for (int d = lane; d < E; d += 64) stf<P>(orow + d, column(0, d) * c);
+  } else {
+    float v[BSA_MAXC], ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < BSA_MAXC; ++c) {
+      const int d = lane + 64 * c;
+      if (64 * c < E) {                                  // uniform
+        const float o = d < E ? column(0, d) - form.lambda * column(1, d) : 0.f;
+        v[c] = o;
+        ss += o * o;
+      }
+    }
+    ss = wave_sum(ss);
+    const float c0 = out_scale * gt / sqrtf(ss / (float)E + form.eps);
+#pragma unroll
+    for (int c = 0; c < BSA_MAXC; ++c)
+      if (lane + 64 * c < E) stf<P>(orow + lane + 64 * c, v[c] * c0);
   }
+}
+
+static inline bool form_ok(const UmbAttnForm* f) { return !f || ((f->maps == 1 || f->maps == 2) && f->chunk >= 0); }
+
+extern "C" int umb_attn_prep(float* q, const UmbPagedKV* kv, const float* proj, int ld, int append, const void* w_q, const void* w_k,
+                             int norm_qk, int norm_v, const int* pos, const int* slot, const float* freq, int rot_dims, int layout,
+                             float rot_mult, int T, int H, int G, int D, int E, int maps, float temp_coef, int temp_every, float eps,
+                             int dtype, hipStream_t st) {
+  if (T < 1 || H < 1 || G < 1 || H % G || D < 1 || E < 1 || maps < 1 || maps > 2 || rot_dims < 0 || rot_dims > D || (rot_dims & 1) ||
+      (rot_dims && !freq) || layout < 0 || layout > 1 || !q || (append && !bsa_kv_ok(kv)) || !proj || !pos || !slot ||
+      ld < maps * H * D + (append ? maps * G * D + G * E : 0))
+    return UMB_EINVAL;
+  AttnPrep a{maps * H, append ? maps * G : 0, G, append ? G : 0, D, E, maps, norm_qk, norm_v, rot_dims, layout, rot_mult,
+             temp_coef, temp_every, eps};
+  const UmbPagedKV none{};
+  const long items = (long)T * (a.HQ + a.GK + a.GV);
+  DISPATCH_SEQ_DTYPE(dtype, {
+    typedef typename El<P>::type El_;
+    hipLaunchKernelGGL(attn_prep_kernel<P>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st, q, append ? *kv : none, proj, ld,
+                       (const El_*)w_q, (const El_*)w_k, pos, slot, freq, T, a);
+  })
+  UMB_LAUNCH_CHECK();
+  return UMB_OK;
 }
 
 extern "C" int umb_bsa_prep(float* q, const UmbPagedKV* kv, const float* proj, int ld, const void* w_q, const void* w_k,
                             const int* pos, const int* slot, int T, int H, int G, int D, int E, float temp_coef, int temp_every,
                             float eps, int dtype, hipStream_t st) {
-  if (T < 1 || H < 1 || G < 1 || H % G || D < 1 || E < 1 || !q || !bsa_kv_ok(kv) || !proj || !pos || !slot ||
-      ld < H * D + G * D + G * E)
+  return umb_attn_prep(q, kv, proj, ld, 1, w_q, w_k, 1, 1, pos, slot, nullptr, 0, 0, 1.f, T, H, G, D, E, 1, temp_coef, temp_every, eps,
+                       dtype, st);
+}
+
+template <typename P, int RH, int NC, int NW, int MAPS>
+static int bsa_launch(dim3 grid, size_t lds, hipStream_t st, void* out, int ldo, const float* q, const UmbPagedKV& kv,
+                      const float* proj, int ld, int gate_col, const float* bias, int n_dist, const int* pos, const int* slot, int H,
+                      int G, int D, int E, int window, float scale, float out_scale, float softcap, const UmbAttnForm& form,
+                      float* scratch, int nsplit) {
+  typedef typename El<P>::type El_;
+  if (ensure_dynamic_lds<bsa_attend_kernel<P, RH, NC, NW, MAPS>>(lds) != UMB_OK) return UMB_EHIP;
+  hipLaunchKernelGGL((bsa_attend_kernel<P, RH, NC, NW, MAPS>), grid, dim3(NW * 64), lds, st, (El_*)out, ldo, q, kv, proj, ld, gate_col,
+                     bias, n_dist, pos, slot, H, G, D, E, window, scale, out_scale, softcap, form, scratch, nsplit);
+  return UMB_OK;
+}
+
+extern "C" int umb_attn_attend(void* out, int ldo, const float* q, const UmbPagedKV* kv, const float* proj, int ld, int gate_col,
+                               const float* bias, int n_dist, const int* pos, const int* slot, int T, int H, int G, int D, int E,
+                               int window, float scale, float out_scale, float softcap, const UmbAttnForm* form_, float* scratch,
+                               long scratch_floats, int dtype, hipStream_t st) {
+  if (T < 1 || H < 1 || G < 1 || H % G || D < 1 || E < 1 || E > 64 * BSA_MAXC || window < 1 || !out || !q || !bsa_kv_ok(kv) ||
+      !pos || !slot || ldo < H * E || (bias && n_dist < 1) || (gate_col >= 0 && (!proj || ld < gate_col + H)) || !form_ok(form_))
     return UMB_EINVAL;
-  const long items = (long)T * (H + 2 * G);
+  const UmbAttnForm form = form_ ? *form_ : UmbAttnForm{1, 0, nullptr, 0.f, 0.f};
+  const int maps = form.maps;
+  const int hpg = H / G, nc = (E + 63) / 64;
+  const int Dp = (D + 3) & ~3, Ep = (E + 3) & ~3, Mp = Dp > Ep ? Dp : Ep;
+  // rows (head, map) of one workgroup: query heads of one key/value head, as many as divide the group and fit the register budget
+  int rh = nc <= 2 ? 8 : (nc <= 4 ? 4 : 2);
+  while (rh > maps && hpg % (rh / maps)) rh >>= 1;
+  // A handful of (token, head block) items leaves most of the chip idle while each walks all its keys: with scratch for the
+  // partial results the keys of an item are dealt to several workgroups (whole groups of four 64-key rounds by number, so the
+  // order of every sum is a function of the position and of the step's row count only) and merged by a second launch.
+  const int hblocks = H * maps / rh;
+  const long items = (long)T * hblocks;
+  int nsplit = 1;
+  if (scratch && items <= 64) {                          // fewer than ~2048 waves in all with sixteen waves per item
+    nsplit = (int)(512 / items) < 16 ? (int)(512 / items) : 16;
+    // keys of one chunk only: no more workgroups than there can be groups of four rounds
+    if (form.chunk > 0 && nsplit > (form.chunk + 255) / 256) nsplit = (form.chunk + 255) / 256;
+    while (nsplit > 1 && (long)T * H * maps * nsplit * (E + 2) > scratch_floats) nsplit >>= 1;
+  }
+  const dim3 grid(T, hblocks, nsplit);
+  int nw = (nsplit > 1 || items >= 1024) ? 4 : 16;
+  auto lds_of = [&](int w) { return ((size_t)w * rh * Mp + (size_t)w * 2 * rh + (size_t)w * (rh * 64 + 128)) * sizeof(float); };
+  if (nw == 16 && lds_of(16) > 128 * 1024) nw = 4;
+  if (lds_of(nw) > 160 * 1024) return UMB_EINVAL;
+  const size_t lds = lds_of(nw);
+#define BSA_GO(RH, NC, NW, MAPS)                                                                                             \
+  SEQ_TRY_((bsa_launch<P, RH, NC, NW, MAPS>(grid, lds, st, out, ldo, q, *kv, proj, ld, gate_col, bias, n_dist, pos, slot, H, G, D,   \
+                                           E, window, scale, out_scale, softcap, form, scratch, nsplit)))
+#define SEQ_TRY_(call) do { const int rc__ = (call); if (rc__ != UMB_OK) return rc__; } while (0)
+#define BSA_NW(RH, NC, MAPS)                                                                                                 \
+  do { if (nw == 16) BSA_GO(RH, NC, 16, MAPS); else BSA_GO(RH, NC, 4, MAPS); } while (0)
+#define BSA_RH(NC)                                                                                                           \
+  do {                                                                                                                       \
+    if (maps == 2) { if (rh == 8) BSA_NW(8, NC, 2); else if (rh == 4) BSA_NW(4, NC, 2); else BSA_NW(2, NC, 2); }              \
+    else if (rh == 8) BSA_NW(8, NC, 1); else if (rh == 4) BSA_NW(4, NC, 1); else if (rh == 2) BSA_NW(2, NC, 1);               \
+    else BSA_NW(1, NC, 1);                                                                                                   \
+  } while (0)
   DISPATCH_SEQ_DTYPE(dtype, {
     typedef typename El<P>::type El_;
-    hipLaunchKernelGGL(bsa_prep_kernel<P>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st, q, *kv, proj, ld, (const El_*)w_q,
-                       (const El_*)w_k, pos, slot, T, H, G, D, E, temp_coef, temp_every, eps);
+    if (nc <= 1) BSA_RH(1);
+    else if (nc <= 2) BSA_RH(2);
+    else if (nc <= 4) {
+      if (maps == 2) { if (rh == 4) BSA_NW(4, 4, 2); else BSA_NW(2, 4, 2); }
+      else if (rh == 4) BSA_NW(4, 4, 1); else if (rh == 2) BSA_NW(2, 4, 1); else BSA_NW(1, 4, 1);
+    } else {
+      if (maps == 2) BSA_NW(2, 8, 2); else if (rh == 2) BSA_NW(2, 8, 1); else BSA_NW(1, 8, 1);
+    }
+    if (nsplit > 1) {
+      if (maps == 2)
+        hipLaunchKernelGGL((bsa_merge_kernel<P, 2>), dim3(T, H), dim3(64), 0, st, (El_*)out, ldo, scratch, proj, ld, gate_col, H, E,
+                           nsplit, out_scale, form);
+      else
+        hipLaunchKernelGGL((bsa_merge_kernel<P, 1>), dim3(T, H), dim3(64), 0, st, (El_*)out, ldo, scratch, proj, ld, gate_col, H, E,
+                           nsplit, out_scale, form);
+    }
   })
+#undef BSA_RH
+#undef BSA_NW
+#undef BSA_GO
+#undef SEQ_TRY_
   UMB_LAUNCH_CHECK();
   return UMB_OK;
 }
@@ -259,54 +466,8 @@ extern "C" int umb_bsa_attend(void* out, int ldo, const float* q, const UmbPaged
                               const float* bias, int n_dist, const int* pos, const int* slot, int T, int H, int G, int D, int E,
                               int window, float scale, float out_scale, float softcap, float* scratch, long scratch_floats,
                               int dtype, hipStream_t st) {
-  if (T < 1 || H < 1 || G < 1 || H % G || D < 1 || E < 1 || E > 64 * BSA_MAXC || window < 1 || !out || !q || !bsa_kv_ok(kv) ||
-      !pos || !slot || ldo < H * E || (bias && n_dist < 1) || (gate_col >= 0 && (!proj || ld < gate_col + H)))
-    return UMB_EINVAL;
-  const int hpg = H / G, nc = (E + 63) / 64;
-  const int Dp = (D + 3) & ~3, Ep = (E + 3) & ~3, Mp = Dp > Ep ? Dp : Ep;
-  // heads of one workgroup: query heads of one key/value head, as many as divide the group and fit the register budget
-  int rh = nc <= 2 ? 8 : (nc <= 4 ? 4 : 2);
-  while (rh > 1 && hpg % rh) rh >>= 1;
-  // A handful of (token, head block) items leaves most of the chip idle while each walks all its keys: with scratch for the
-  // partial results the keys of an item are dealt to several workgroups (whole groups of four 64-key rounds by number, so the
-  // order of every sum is a function of the position and of the step's row count only) and merged by a second launch.
-  const long items = (long)T * (H / rh);
-  int nsplit = 1;
-  if (scratch && items <= 64) {                          // fewer than ~2048 waves in all with sixteen waves per item
-    nsplit = (int)(512 / items) < 16 ? (int)(512 / items) : 16;
-    while (nsplit > 1 && (long)T * H * nsplit * (E + 2) > scratch_floats) nsplit >>= 1;
-  }
-  const dim3 grid(T, H / rh, nsplit);
-  int nw = (nsplit > 1 || items >= 1024) ? 4 : 16;
-  auto lds_of = [&](int w) { return ((size_t)w * rh * Mp + (size_t)w * 2 * rh + (size_t)w * (rh * 64 + 128)) * sizeof(float); };
-  if (nw == 16 && lds_of(16) > 128 * 1024) nw = 4;
-  if (lds_of(nw) > 160 * 1024) return UMB_EINVAL;
-  const size_t lds = lds_of(nw);
-#define BSA_LAUNCH(RH, NC, NW)                                                                                              \
-  do {                                                                                                                      \
-    if (ensure_dynamic_lds<bsa_attend_kernel<P, RH, NC, NW>>(lds) != UMB_OK) return UMB_EHIP;                               \
-    hipLaunchKernelGGL((bsa_attend_kernel<P, RH, NC, NW>), grid, dim3(NW * 64), lds, st, (El_*)out, ldo, q, *kv, proj, ld,  \
-                       gate_col, bias, n_dist, pos, slot, H, G, D, E, window, scale, out_scale, softcap, scratch, nsplit);           \
-  } while (0)
-#define BSA_NW(RH, NC)                                                                                                      \
-  if (nw == 16) BSA_LAUNCH(RH, NC, 16); else BSA_LAUNCH(RH, NC, 4)
-#define BSA_RH(NC)                                                                                                          \
-  if (rh == 8) { BSA_NW(8, NC); } else if (rh == 4) { BSA_NW(4, NC); } else if (rh == 2) { BSA_NW(2, NC); } else { BSA_NW(1, NC); }
-  DISPATCH_SEQ_DTYPE(dtype, {
-    typedef typename El<P>::type El_;
-    if (nc <= 1) { BSA_RH(1) }
-    else if (nc <= 2) { BSA_RH(2) }
-    else if (nc <= 4) { if (rh == 4) { BSA_NW(4, 4); } else if (rh == 2) { BSA_NW(2, 4); } else { BSA_NW(1, 4); } }
-    else { if (rh == 2) { BSA_NW(2, 8); } else { BSA_NW(1, 8); } }
-    if (nsplit > 1)
-      hipLaunchKernelGGL(bsa_merge_kernel<P>, dim3(T, H), dim3(64), 0, st, (El_*)out, ldo, scratch, proj, ld, gate_col, H, E, nsplit,
-                         out_scale);
-  })
-#undef BSA_RH
-#undef BSA_NW
-#undef BSA_LAUNCH
-  UMB_LAUNCH_CHECK();
-  return UMB_OK;
+  return umb_attn_attend(out, ldo, q, kv, proj, ld, gate_col, bias, n_dist, pos, slot, T, H, G, D, E, window, scale, out_scale,
+                         softcap, nullptr, scratch, scratch_floats, dtype, st);
 }
 
 // ---- prompt attention on the matrix pipe (16-bit storage; D a multiple of 8, E a multiple of 16).
@@ -327,28 +488,32 @@ template <typename P> __device__ __forceinline__ void split2(float a, float b, u
   lo = pack2<P>(a - P::to_f(ah), b - P::to_f(bh));
 }
 
-template <typename P, int NSM, int NVM, int HPW>
+// HPW rows per wave = HPW / MAPS heads with MAPS maps each; every map has its part of the staged key rows, the value fragments of
+// a step serve all rows
+template <typename P, int NSM, int NVM, int HPW, int MAPS>
 __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ out, int ldo, const float* __restrict__ q,
                                                               UmbPagedKV kv, const float* __restrict__ proj, int ld, int gate_col,
                                                               const float* __restrict__ bias, int n_dist,
                                                               const int* __restrict__ seq_slot, const int* __restrict__ seq_row0,
                                                               const int* __restrict__ seq_pos0, const int* __restrict__ seq_len,
                                                               int H, int G, int D, int E, int window, float scale, float out_scale,
-                                                              float softcap) {
+                                                              float softcap, UmbAttnForm form) {
   extern __shared__ __attribute__((aligned(16))) u16 bsa_lds[];
-  constexpr int NLK = (NSM * 4 + 7) / 8, NLV = (NVM * 2 + 7) / 8;     // 16-byte chunks of a key / value row per staging thread
+  static_assert(HPW % MAPS == 0, "a wave owns whole heads");
+  constexpr int HW = HPW / MAPS;                      // heads per wave
+  constexpr int NLK = (NSM * 4 * MAPS + 7) / 8, NLV = (NVM * 2 + 7) / 8;     // 16-byte chunks of a key / value row per staging thread
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, j = lane & 15, g4 = lane >> 4;
-  const int LD = D + 8;                               // LDS row stride of the key tile: 16 bytes of padding spread the banks
-  const int ns = (D + 31) >> 5, nv = E >> 4, nck = D >> 3, ncv = E >> 3;
+  const int DK = MAPS * D, LD = DK + 8;               // LDS row stride of the key tile: 16 bytes of padding spread the banks
+  const int ns = (D + 31) >> 5, nv = E >> 4, nck = DK >> 3, ncv = E >> 3;
   constexpr int LT = 36;                              // row stride of the transposed value tile: 32 keys + 8 bytes of padding
   u16* k_s = bsa_lds;                                 // [32][LD]
   u16* v_t = bsa_lds + 32 * LD;                       // [E][LT]
   const int b = blockIdx.y;
   const int n = seq_len[b], q0 = blockIdx.x * 16;
   if (q0 >= n) return;                                // the whole workgroup
-  const int hpg = H / G, hblocks = (hpg + 4 * HPW - 1) / (4 * HPW);
+  const int hpg = H / G, hblocks = (hpg + 4 * HW - 1) / (4 * HW);
   const int g = blockIdx.z / hblocks;
-  const int hl0 = ((blockIdx.z % hblocks) * 4 + wave) * HPW;         // first of the wave's heads inside the group
+  const int hl0 = ((blockIdx.z % hblocks) * 4 + wave) * HW;         // first of the wave's heads inside the group
   const bool active = hl0 < hpg;                      // a wave without heads still stages rows and meets the barriers
   const int slot = seq_slot[b], row0 = seq_row0[b], pos0 = seq_pos0[b];
   const int nq = n - q0 < 16 ? n - q0 : 16;
@@ -356,7 +521,12 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
   const bool q_ok = j < nq;
   const int i_j = i_first + (q_ok ? j : nq - 1);
   const long qrow = row0 + q0 + (q_ok ? j : nq - 1);
-  const int j_lo = i_first - window + 1 > 0 ? i_first - window + 1 : 0;
+  int j_lo = i_first - window + 1 > 0 ? i_first - window + 1 : 0;
+  int c_lo = 0;                                       // first position of the query's own chunk
+  if (form.chunk > 0) {
+    j_lo = max(j_lo, i_first / form.chunk * form.chunk);
+    c_lo = i_j / form.chunk * form.chunk;
+  }
   const int total = i_last - j_lo + 1;
   const float scale2 = scale * BSA_LOG2E;
   const u16* kbase = reinterpret_cast<const u16*>(kv.k);
@@ -368,9 +538,9 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
   int hd[HPW];
 #pragma unroll
   for (int hh = 0; hh < HPW; ++hh) {
-    h_ok[hh] = hl0 + hh < hpg;
-    hd[hh] = g * hpg + (h_ok[hh] ? hl0 + hh : hpg - 1);
-    const float* qr = q + (qrow * H + hd[hh]) * D;
+    h_ok[hh] = hl0 + hh / MAPS < hpg;
+    hd[hh] = g * hpg + (h_ok[hh] ? hl0 + hh / MAPS : hpg - 1);
+    const float* qr = q + ((qrow * H + hd[hh]) * MAPS + hh % MAPS) * D;
 #pragma unroll
     for (int s = 0; s < NSM; ++s) {
       const int d = 32 * s + 8 * g4;
@@ -398,7 +568,7 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
   auto fetch = [&](int base) {
     const int kx = base + sm;
     const bool ok = kx < total;
-    const long offk = ok ? pkv_tok(kv, slot, j_lo + kx, g, G, D) : 0;
+    const long offk = ok ? pkv_tok(kv, slot, j_lo + kx, g, G, DK) : 0;
     const long offv = ok ? pkv_tok(kv, slot, j_lo + kx, g, G, E) : 0;
 #pragma unroll
     for (int u = 0; u < NLK; ++u) {
@@ -439,7 +609,7 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
       const int jt = j_lo + base + 16 * (e >> 2) + 4 * g4 + (e & 3);
-      vis[e] = q_ok && jt <= i_j && jt > i_j - window;
+      vis[e] = q_ok && jt <= i_j && jt > i_j - window && jt >= c_lo;
       const int dd = i_j - jt;
       di[e] = dd < 0 ? 0 : (dd < n_dist ? dd : n_dist - 1);
     }
@@ -458,11 +628,14 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
       for (int s = 0; s < NSM; ++s) {
         const int d = 32 * s + 8 * g4;
         if (s < ns) {
-          const u32x4 kf = d < D ? *reinterpret_cast<const u32x4*>(kr + d) : u32x4{0u, 0u, 0u, 0u};
 #pragma unroll
-          for (int hh = 0; hh < HPW; ++hh) {
-            sc2[hh][u] = P::mfma(kf, ql[hh][s], sc2[hh][u]);
-            sc2[hh][u] = P::mfma(kf, qh[hh][s], sc2[hh][u]);
+          for (int mp = 0; mp < MAPS; ++mp) {
+            const u32x4 kf = d < D ? *reinterpret_cast<const u32x4*>(kr + mp * D + d) : u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+            for (int hh = mp; hh < HPW; hh += MAPS) {
+              sc2[hh][u] = P::mfma(kf, ql[hh][s], sc2[hh][u]);
+              sc2[hh][u] = P::mfma(kf, qh[hh][s], sc2[hh][u]);
+            }
           }
         }
       }
@@ -524,10 +697,32 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
   // lane holds O^T[d = 16 dt + 4 g4 + rr][query j]
   if (q_ok && active) {
 #pragma unroll
-    for (int hh = 0; hh < HPW; ++hh) {
+    for (int hh = 0; hh < HPW; hh += MAPS) {
       if (!h_ok[hh]) continue;
       const float gt = gate_col >= 0 ? 1.f / (1.f + expf(-proj[qrow * ld + gate_col + hd[hh]])) : 1.f;
-      const float inv = out_scale * gt / l_run[hh];
+      float l[MAPS];
+#pragma unroll
+      for (int mp = 0; mp < MAPS; ++mp)
+        l[mp] = l_run[hh + mp] + (form.sink ? __builtin_amdgcn_exp2f(form.sink[hd[hh]] * BSA_LOG2E - m_run[hh + mp]) : 0.f);
+      float inv = out_scale * gt / l[0];
+      if constexpr (MAPS == 2) {                      // o = a1 - lambda a2 over the root mean square of the head's E columns
+        const float i1 = 1.f / l[0], i2 = form.lambda / l[1];
+        float ss = 0.f;
+#pragma unroll
+        for (int dt = 0; dt < NVM; ++dt) {
+          if (dt < nv) {
+#pragma unroll
+            for (int rr = 0; rr < 4; ++rr) {
+              const float v = o[hh][dt][rr] * i1 - o[hh + 1][dt][rr] * i2;
+              o[hh][dt][rr] = v;
+              ss += v * v;
+            }
+          }
+        }
+        ss += __shfl_xor(ss, 16, 64);                 // the query's column quads: lanes j, j + 16, j + 32, j + 48 (all active)
+        ss += __shfl_xor(ss, 32, 64);
+        inv = out_scale * gt / sqrtf(ss / (float)E + form.eps);
+      }
       u16* orow = out + qrow * ldo + (long)hd[hh] * E;
 #pragma unroll
       for (int dt = 0; dt < NVM; ++dt) {
@@ -545,34 +740,45 @@ extern "C" int umb_bsa_attend_tiled_ok(int H, int G, int D, int E, int dtype) {
          E >= 16 && E % 16 == 0 && E <= 256;
 }
 
-extern "C" int umb_bsa_attend_tiled(void* out, int ldo, const float* q, const UmbPagedKV* kv, const float* proj, int ld,
-                                    int gate_col, const float* bias, int n_dist, const int* seq_slot, const int* seq_row0,
-                                    const int* seq_pos0, const int* seq_len, int B, int max_len, int H, int G, int D, int E,
-                                    int window, float scale, float out_scale, float softcap, int dtype, hipStream_t st) {
+extern "C" int umb_attn_attend_tiled(void* out, int ldo, const float* q, const UmbPagedKV* kv, const float* proj, int ld,
+                                     int gate_col, const float* bias, int n_dist, const int* seq_slot, const int* seq_row0,
+                                     const int* seq_pos0, const int* seq_len, int B, int max_len, int H, int G, int D, int E,
+                                     int window, float scale, float out_scale, float softcap, const UmbAttnForm* form_, int dtype,
+                                     hipStream_t st) {
   if (B < 1 || B > 65535 || max_len < 1 || window < 1 || !out || !q || !bsa_kv_ok(kv) || !seq_slot || !seq_row0 || !seq_pos0 ||
       !seq_len || ldo < H * E || (bias && n_dist < 1) || (gate_col >= 0 && (!proj || ld < gate_col + H)) ||
-      !umb_bsa_attend_tiled_ok(H, G, D, E, dtype))
+      !umb_bsa_attend_tiled_ok(H, G, D, E, dtype) || !form_ok(form_))
     return UMB_EINVAL;
   if (!bias) n_dist = 1;
-  const int hpg = H / G;
-  const size_t lds = ((size_t)32 * (D + 8) + (size_t)E * 36) * sizeof(u16);
-#define BSA_MFMA(NSM, NVM, HPW)                                                                                            \
+  const UmbAttnForm form = form_ ? *form_ : UmbAttnForm{1, 0, nullptr, 0.f, 0.f};
+  const int hpg = H / G, maps = form.maps;
+  const size_t lds = ((size_t)32 * (maps * D + 8) + (size_t)E * 36) * sizeof(u16);
+#define BSA_MFMA(NSM, NVM, HPW, MAPS)                                                                                      \
   do {                                                                                                                     \
-    const int hblocks = (hpg + 4 * HPW - 1) / (4 * HPW);                                                                   \
+    const int hblocks = (hpg + 4 * (HPW / MAPS) - 1) / (4 * (HPW / MAPS));                                                 \
     if ((long)G * hblocks > 65535) return UMB_EINVAL;                                                                      \
     const dim3 grid((max_len + 15) / 16, B, G * hblocks);                                                                  \
-    if (ensure_dynamic_lds<bsa_attend_mfma_kernel<P, NSM, NVM, HPW>>(lds) != UMB_OK) return UMB_EHIP;                      \
-    hipLaunchKernelGGL((bsa_attend_mfma_kernel<P, NSM, NVM, HPW>), grid, dim3(256), lds, st, (u16*)out, ldo, q, *kv, proj, \
-                       ld, gate_col, bias, n_dist, seq_slot, seq_row0, seq_pos0, seq_len, H, G, D, E, window, scale,       \
-                       out_scale, softcap);                                                                                \
+    if (ensure_dynamic_lds<bsa_attend_mfma_kernel<P, NSM, NVM, HPW, MAPS>>(lds) != UMB_OK) return UMB_EHIP;                \
+    hipLaunchKernelGGL((bsa_attend_mfma_kernel<P, NSM, NVM, HPW, MAPS>), grid, dim3(256), lds, st, (u16*)out, ldo, q, *kv, \
+                       proj, ld, gate_col, bias, n_dist, seq_slot, seq_row0, seq_pos0, seq_len, H, G, D, E, window, scale, \
+                       out_scale, softcap, form);                                                                          \
   } while (0)
 #define BSA_MFMA_SHAPE()                                                                                                   \
-  if (D <= 128 && E <= 128) { if (hpg > 4) BSA_MFMA(4, 8, 2); else BSA_MFMA(4, 8, 1); }                                    \
-  else BSA_MFMA(8, 16, 1)
+  if (maps == 2) { if (D <= 128 && E <= 128) BSA_MFMA(4, 8, 2, 2); else BSA_MFMA(8, 16, 2, 2); }                           \
+  else if (D <= 128 && E <= 128) { if (hpg > 4) BSA_MFMA(4, 8, 2, 1); else BSA_MFMA(4, 8, 1, 1); }                         \
+  else BSA_MFMA(8, 16, 1, 1)
   if (dtype == UMB_SEQ_BF16) { using P = BF16; BSA_MFMA_SHAPE(); }
   else { using P = F16; BSA_MFMA_SHAPE(); }
 #undef BSA_MFMA_SHAPE
 #undef BSA_MFMA
   UMB_LAUNCH_CHECK();
   return UMB_OK;
+}
+
+extern "C" int umb_bsa_attend_tiled(void* out, int ldo, const float* q, const UmbPagedKV* kv, const float* proj, int ld,
+                                    int gate_col, const float* bias, int n_dist, const int* seq_slot, const int* seq_row0,
+                                    const int* seq_pos0, const int* seq_len, int B, int max_len, int H, int G, int D, int E,
+                                    int window, float scale, float out_scale, float softcap, int dtype, hipStream_t st) {
+  return umb_attn_attend_tiled(out, ldo, q, kv, proj, ld, gate_col, bias, n_dist, seq_slot, seq_row0, seq_pos0, seq_len, B, max_len, H,
+                               G, D, E, window, scale, out_scale, softcap, nullptr, dtype, st);
 }

@@ -13,6 +13,9 @@
 //     convolved attention beside a matrix memory (one fused proj GEMM, one out GEMM over [a | b]):
 //                convolution + whole-row norms + rotary + append | ring | attend (capped scores)  ||  gates + running maximum |
 //                scaled queries + widened values | scan | stabilised division + per-head norm + sigmoid gate
+//     differential attention: proj GEMM ([q | k | v], or [q] over another layer's store) | rotary + append | attend + combine | out GEMM
+//     attention with a sink beside a gated delta rule (one fused proj GEMM): norms + append | attend  ||  convolution + unit norms +
+//                gates | ring | chunk solve | chunk scan (single tokens: one launch) | per-head norm * SiLU gate | two out GEMMs | pair seam
 // Stacks whose two sublayers read the SAME residual (UmbSeqModel.block = UMB_BLOCK_PARALLEL) run mixer and feed-forward from two
 // normed inputs and meet in one seam per layer; a layer may ask for the embedding row to be added again in front of it.
 // Models with several residual streams (UmbSeqModel.streams >= 1) use the stream seam instead: write of the sublayer behind
@@ -262,6 +265,70 @@ static int mix_attn_mlstm(const UmbSeqModel* m, const UmbSeqLayer& ly, const Umb
   return umb_head_gate(right, ldo, ws->o, Pp, Em, mrun, ws->proj, ld, mg, ly.m_norm, 1, 1, T, Hm, Em, m->eps, ly.mix_scale_b, dt, st);
 }
 
+// the two places attention mixers meet the keys: the matrix pipe for steps that bring stretches, the vector pipe otherwise
+static int attend(const UmbSeqLayer& ly, void* out, const float* q, const UmbSeqStep* s, int H, int G, int D, int E, int window,
+                  float out_scale, const UmbAttnForm& form, float* scratch, long scratch_floats, int dt, hipStream_t st) {
+  if (s->max_len >= 16 && umb_bsa_attend_tiled_ok(H, G, D, E, dt))
+    return umb_attn_attend_tiled(out, H * E, q, &ly.kv, nullptr, 0, -1, nullptr, 0, s->seq_slot, s->seq_row0, s->seq_pos0, s->seq_len, s->B,
+                                 s->max_len, H, G, D, E, window, ly.scale, out_scale, 0.f, &form, dt, st);
+  return umb_attn_attend(out, H * E, q, &ly.kv, nullptr, 0, -1, nullptr, 0, s->pos, s->slot, s->T, H, G, D, E, window, ly.scale, out_scale,
+                         0.f, &form, scratch_floats > 0 ? scratch : nullptr, scratch_floats, dt, st);
+}
+
+// differential attention: two maps per head over the same values; with kv_shared the keys and values are another layer's
+static int mix_diff_attn(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWork* ws, const UmbSeqStep* s, hipStream_t st) {
+  const int T = s->T, dt = m->dtype, ld = ly.proj.N, H = ly.heads, G = ly.kv_heads, D = ly.dim, E = ly.vdim;
+  if (H < 1 || G < 1 || ld != 2 * H * D + (ly.kv_shared ? 0 : 2 * G * D + G * E) || ly.out.K != H * E) return UMB_EINVAL;
+  float* q = ws->aux;                                        // [T][H][2][D] | scratch
+  float* spare = q + al4((long)T * 2 * H * D);
+  SEQ_TRY(umb_attn_prep(q, &ly.kv, ws->proj, ld, !ly.kv_shared, nullptr, nullptr, 0, 0, s->pos, s->slot, ly.rot_freq, ly.rot_dims,
+                        ly.rot_layout, ly.rot_mult, T, H, G, D, E, 2, 0.f, 0, m->eps, dt, st));
+  const UmbAttnForm form{2, ly.chunk, nullptr, ly.diff_lambda, m->eps};
+  return attend(ly, ws->mix, q, s, H, G, D, E, ly.window, ly.out_mult, form, spare, ws->aux_floats - (long)(spare - ws->aux), dt, st);
+}
+
+static inline int up16(int n) { return (n + 15) & ~15; }
+// elements between the two mixers' outputs in ws->mix (rows of the second start 16-byte aligned)
+static inline long mix_right(const UmbSeqLayer& ly, int T) { return ((long)T * ly.heads * ly.vdim + 63) & ~63L; }
+
+// attention with a sink beside a gated delta rule; both read the projection of the same input, each leaves its own rows in ws->mix
+// ([T][heads vdim], then [T][s_heads s_vdim]) for its own output projection
+static int mix_attn_delta(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWork* ws, const UmbSeqStep* s, hipStream_t st) {
+  const int T = s->T, dt = m->dtype, ld = ly.proj.N, H = ly.heads, G = ly.kv_heads, D = ly.dim, E = ly.vdim;
+  const int Hk = ly.s_groups, Hv = ly.s_heads, Ds = ly.s_state, Es = ly.s_vdim;
+  if (H < 1 || G < 1 || Hk < 1 || Hv < 1) return UMB_EINVAL;
+  const int col0 = H * D + G * D + G * E, C = 2 * Hk * Ds + Hv * Es;
+  if (ld != col0 + C + Hv * Es + 2 * Hv || ly.out.K != H * E || ly.out2.K != Hv * Es || !ly.state) return UMB_EINVAL;
+  float* q = ws->aux;                                        // [T][H D] | dq | dk | dv | beta | log g | scratch
+  float* spare = q + al4((long)T * H * D);
+  SEQ_TRY(umb_attn_prep(q, &ly.kv, ws->proj, ld, 1, ly.q_norm, ly.k_norm, 1, 0, s->pos, s->slot, nullptr, 0, 0, 1.f, T, H, G, D, E, 1, 0.f, 0,
+                        m->eps, dt, st));
+  const UmbAttnForm form{1, 0, ly.attn_sink, 0.f, 0.f};
+  SEQ_TRY(attend(ly, ws->mix, q, s, H, G, D, E, ly.window, 1.f, form, spare, ws->aux_floats - (long)(spare - ws->aux), dt, st));
+  if (s->max_len == 1)
+    SEQ_TRY(umb_delta_step(ws->o, ly.state, ws->proj, ld, col0, ly.s_conv, ly.s_conv_state, ly.s_dt_bias, ly.s_a_log, s->pos, s->slot, T, Hk,
+                           Hv, Ds, Es, ly.s_taps, dt, st));
+  else {
+    const int ldqk = Hk * up16(Ds);
+    float* dq = spare;
+    float* dk = dq + (long)T * ldqk;
+    float* dv = dk + (long)T * ldqk;
+    float* beta = dv + al4((long)T * Hv * Es);
+    float* lg = beta + al4((long)T * Hv);
+    float* scratch = lg + al4((long)T * Hv);
+    const long scratch_floats = ws->aux_floats - (long)(scratch - ws->aux);
+    if (scratch_floats < umb_delta_scan_floats(T, Hv, Ds, Es)) return UMB_EINVAL;
+    SEQ_TRY(umb_delta_prep(dq, dk, ldqk, dv, beta, lg, ws->proj, ld, col0, ly.s_conv, ly.s_conv_state, ly.s_dt_bias, ly.s_a_log, s->pos,
+                           s->slot, T, Hk, Hv, Ds, Es, ly.s_taps, dt, st));
+    SEQ_TRY(umb_ssd_conv_update(ly.s_conv_state, ws->proj, ld, col0, s->seq_slot, s->seq_row0, s->seq_pos0, s->seq_len, s->B, C,
+                                ly.s_taps + 1, st));
+    SEQ_TRY(umb_delta_scan(ws->o, ly.state, dq, dk, ldqk, dv, beta, lg, s->seq_slot, s->seq_row0, s->seq_pos0, s->seq_len, T, s->B, s->max_len,
+                           Hk, Hv, Ds, Es, scratch, scratch_floats, st));
+  }
+  void* right = static_cast<char*>(ws->mix) + mix_right(ly, T) * seq_elem_bytes(dt);
+  return umb_head_gate(right, Hv * Es, ws->o, Es, -1, nullptr, ws->proj, ld, col0 + C, ly.s_norm, 0, 0, T, Hv, Es, m->eps, 1.f, dt, st);
+}
+
 // the mixer of one layer: from the fused projection in ws->proj to the row ws->mix that the output projection reads
 static int run_mixer(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWork* ws, const UmbSeqStep* s, hipStream_t st) {
   const int T = s->T, dt = m->dtype, ld = ly.proj.N;
@@ -313,6 +380,11 @@ static int run_mixer(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWo
     SEQ_TRY(mix_retention(m, ly, ws, s, st));
   } else if (ly.kind == UMB_MIX_ATTN_MLSTM) {
     SEQ_TRY(mix_attn_mlstm(m, ly, ws, s, st));
+  } else if (ly.kind == UMB_MIX_DIFF_ATTN) {
+    SEQ_TRY(mix_diff_attn(m, ly, ws, s, st));
+  } else if (ly.kind == UMB_MIX_ATTN_DELTA) {
+    if (m->block == UMB_BLOCK_PARALLEL || m->streams >= 1 || m->groups != 1 || !ws->y2) return UMB_EINVAL;      // its seam is a single stream's
+    SEQ_TRY(mix_attn_delta(m, ly, ws, s, st));
   } else {
     return UMB_EINVAL;
   }
@@ -374,7 +446,7 @@ extern "C" int umb_seq_forward(const UmbSeqModel* m, const UmbSeqWork* ws, const
     SEQ_TRY(umb_hc_embed(ws->x, ws->h, m->embed, s->tokens, m->embed_scale, m->layers[0].hc1_in, m->layers[0].norm1,
                          m->norm_offset, T, W, m->V, S, eps, dt, st));
   } else if (m->layers[0].norm1)
-    SEQ_TRY(umb_seq_embed_norm(ws->x, ws->h, m->embed, s->tokens, m->layers[0].norm1, T, W, m->V, groups, eps, dt, st));
+    SEQ_TRY(umb_seq_embed_norm(ws->x, ws->h, m->embed, s->tokens, m->embed_scale, m->layers[0].norm1, T, W, m->V, groups, eps, dt, st));
   else
     SEQ_TRY(umb_seq_embed(ws->x, m->embed, s->tokens, m->embed_scale, T, W, m->V, dt, st));
   bool h_ready = false;
@@ -401,8 +473,15 @@ extern "C" int umb_seq_forward(const UmbSeqModel* m, const UmbSeqWork* ws, const
       continue;
     }
     const void* next = ly.has_mlp ? ly.norm2 : first_norm_of(m, l + 1);
-    SEQ_TRY(seam(m, ws, s, ly.norm1b, next, ly.has_mlp ? ly.canon2 : (nl ? nl->canon1 : nullptr),
-                 ly.has_mlp ? ly.canon_state2 : (nl ? nl->canon_state1 : nullptr), &h_ready, st));
+    if (ly.kind == UMB_MIX_ATTN_DELTA) {
+      const void* right = static_cast<char*>(ws->mix) + mix_right(ly, T) * seq_elem_bytes(dt);
+      SEQ_TRY(lin(ly.out2, ws->y2, right, T, 0, dt, st));
+      SEQ_TRY(umb_seq_pair_resid_norm(ws->x, ws->h, ws->y, ws->y2, ly.out_norm_a, ly.out_norm_b, ly.pair_coef, ly.norm1b, next, T, W, eps, dt,
+                                      st));
+      h_ready = false;
+    } else
+      SEQ_TRY(seam(m, ws, s, ly.norm1b, next, ly.has_mlp ? ly.canon2 : (nl ? nl->canon1 : nullptr),
+  ly.has_mlp ? ly.canon_state2 : (nl ? nl->canon_state1 : nullptr), &h_ready, st));
     if (ly.has_mlp) {
       SEQ_TRY(sublayer_input(m, ws, s, ly.norm2, ly.canon2, ly.canon_state2, h_ready, st));
       SEQ_TRY(feed_forward(m, ly, ws, s, ws->h, ws->y, st));

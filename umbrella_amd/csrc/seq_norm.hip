@@ -33,8 +33,9 @@ __global__ __launch_bounds__(256) void group_norm_kernel(float* __restrict__ out
 template <typename P>
 __global__ __launch_bounds__(256) void embed_norm_kernel(float* __restrict__ x, typename El<P>::type* __restrict__ h,
                                                          const typename El<P>::type* __restrict__ embed,
-                                                         const int* __restrict__ tokens, const typename El<P>::type* __restrict__ w,
-                                                         int W, int V, int groups, float eps) {
+                                                         const int* __restrict__ tokens, float scale,
+                                                         const typename El<P>::type* __restrict__ w, int W, int V, int groups,
+                                                         float eps) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int grp = blockIdx.y * 4 + wave;
   if (grp >= groups) return;
@@ -44,10 +45,10 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(float* __restrict__ x, 
   const typename El<P>::type* er = embed + (long)tok * W + (long)grp * gs;
   const long o = (long)t * W + (long)grp * gs;
   float ss = 0.f;
-  for (int i = lane; i < gs; i += 64) { const float v = ldf<P>(er + i); x[o + i] = v; ss += v * v; }
+  for (int i = lane; i < gs; i += 64) { const float v = ldf<P>(er + i) * scale; x[o + i] = v; ss += v * v; }
   ss = wave_sum(ss);
   const float f = 1.f / sqrtf(ss / (float)gs + eps);
-  for (int i = lane; i < gs; i += 64) stf<P>(h + o + i, ldf<P>(er + i) * f * ldf<P>(w + grp * gs + i));
+  for (int i = lane; i < gs; i += 64) stf<P>(h + o + i, ldf<P>(er + i) * scale * f * ldf<P>(w + grp * gs + i));
 }
 
 // values of one (row, group) held by a wave: lane owns elements lane + 64 j.  RV = 0: the group is longer than the register
@@ -233,6 +234,86 @@ __global__ __launch_bounds__(256) void seam_canon_step_kernel(float* __restrict_
   if (S > 0) st[(long)(p % S) * W] = xn;
 }
 
+// The seam behind a mixer that is two mixers side by side: m = coef (norm(y1) w1 + norm(y2) w2), then x <- x + norm(m) w_post and,
+// with w_next, h = norm(x) w_next.  Plain RMS norms over the row; one workgroup per token, the row in registers between the three
+// sums (EPT elements per thread; 0: a long row, re-read from memory).
+template <typename P, int EPT>
+__global__ __launch_bounds__(256) void pair_resid_norm_kernel(float* __restrict__ x, typename El<P>::type* __restrict__ h,
+                                                              const float* __restrict__ y1, const float* __restrict__ y2,
+                                                              const typename El<P>::type* __restrict__ w1,
+                                                              const typename El<P>::type* __restrict__ w2, float coef,
+                                                              const typename El<P>::type* __restrict__ w_post,
+                                                              const typename El<P>::type* __restrict__ w_next, int W, float eps) {
+  __shared__ float red[8], red2[8];
+  const long o = (long)blockIdx.x * W;
+  constexpr int NE = EPT > 0 ? EPT : 1;
+  float a[NE], b[NE], xv[NE], wa[NE], wb[NE], wp[NE];
+  float sa = 0.f, sb = 0.f;
+  if constexpr (EPT > 0) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e, ic = i < W ? i : W - 1;
+      a[e] = y1[o + ic];
+      b[e] = y2[o + ic];
+      xv[e] = x[o + ic];
+      wa[e] = ldf<P>(w1 + ic);
+      wb[e] = ldf<P>(w2 + ic);
+      wp[e] = ldf<P>(w_post + ic);
+    }
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const bool in = (int)threadIdx.x + 256 * e < W;
+      sa += in ? a[e] * a[e] : 0.f;
+      sb += in ? b[e] * b[e] : 0.f;
+    }
+  } else {
+    for (int i = threadIdx.x; i < W; i += 256) { sa += y1[o + i] * y1[o + i]; sb += y2[o + i] * y2[o + i]; }
+  }
+  sa = block_sum<256>(sa, red);
+  sb = block_sum<256>(sb, red2);
+  const float fa = coef / sqrtf(sa / (float)W + eps), fb = coef / sqrtf(sb / (float)W + eps);
+  float sm = 0.f;
+  auto pair_at = [&](int i) { return y1[o + i] * fa * ldf<P>(w1 + i) + y2[o + i] * fb * ldf<P>(w2 + i); };
+  if constexpr (EPT > 0) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      a[e] = a[e] * fa * wa[e] + b[e] * fb * wb[e];
+      sm += (int)threadIdx.x + 256 * e < W ? a[e] * a[e] : 0.f;
+    }
+  } else {
+    for (int i = threadIdx.x; i < W; i += 256) { const float v = pair_at(i); sm += v * v; }
+  }
+  sm = block_sum<256>(sm, red);
+  const float fm = 1.f / sqrtf(sm / (float)W + eps);
+  float sx = 0.f;
+  if constexpr (EPT > 0) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e;
+      xv[e] += a[e] * fm * wp[e];
+      if (i < W) { x[o + i] = xv[e]; sx += xv[e] * xv[e]; }
+    }
+  } else {
+    for (int i = threadIdx.x; i < W; i += 256) {
+      const float v = x[o + i] + pair_at(i) * fm * ldf<P>(w_post + i);
+      x[o + i] = v;
+      sx += v * v;
+    }
+  }
+  if (!w_next) return;
+  sx = block_sum<256>(sx, red2);
+  const float fx = 1.f / sqrtf(sx / (float)W + eps);
+  if constexpr (EPT > 0) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e;
+      if (i < W) stf<P>(h + o + i, xv[e] * fx * ldf<P>(w_next + i));
+    }
+  } else {
+    for (int i = threadIdx.x; i < W; i += 256) stf<P>(h + o + i, x[o + i] * fx * ldf<P>(w_next + i));
+  }
+}
+
 static inline bool norm_args_ok(int T, int W, int groups) { return T >= 1 && W >= 1 && groups >= 1 && W % groups == 0; }
 
 extern "C" int umb_seq_group_norm(float* out_f32, void* out_dt, const float* x, const int* rows, const void* w, int T, int W,
@@ -255,13 +336,13 @@ extern "C" int umb_seq_group_norm(float* out_f32, void* out_dt, const float* x, 
   return UMB_OK;
 }
 
-extern "C" int umb_seq_embed_norm(float* x, void* h, const void* embed, const int* tokens, const void* w, int T, int W, int V,
-                                  int groups, float eps, int dtype, hipStream_t st) {
+extern "C" int umb_seq_embed_norm(float* x, void* h, const void* embed, const int* tokens, float scale, const void* w, int T, int W,
+                                  int V, int groups, float eps, int dtype, hipStream_t st) {
   if (!norm_args_ok(T, W, groups) || !x || !h || !embed || !tokens || !w || V < 1) return UMB_EINVAL;
   DISPATCH_SEQ_DTYPE(dtype, {
     typedef typename El<P>::type E;
     hipLaunchKernelGGL(embed_norm_kernel<P>, dim3(T, (groups + 3) / 4), dim3(256), 0, st, x, (E*)h, (const E*)embed, tokens,
-                       (const E*)w, W, V, groups, eps);
+                       scale, (const E*)w, W, V, groups, eps);
   })
   UMB_LAUNCH_CHECK();
   return UMB_OK;
@@ -320,6 +401,24 @@ extern "C" int umb_seq_resid_canon_step(float* x, void* h, const float* y, const
     }
   })
 #undef SEAM_LAUNCH
+  UMB_LAUNCH_CHECK();
+  return UMB_OK;
+}
+
+extern "C" int umb_seq_pair_resid_norm(float* x, void* h, const float* y1, const float* y2, const void* w1, const void* w2, float coef,
+                                       const void* w_post, const void* w_next, int T, int W, float eps, int dtype, hipStream_t st) {
+  if (!norm_args_ok(T, W, 1) || !x || !y1 || !y2 || !w1 || !w2 || !w_post || (w_next && !h)) return UMB_EINVAL;
+#define PAIR_SEAM(EPT)                                                                                                          \
+  hipLaunchKernelGGL((pair_resid_norm_kernel<P, EPT>), dim3(T), dim3(256), 0, st, x, (E*)h, y1, y2, (const E*)w1, (const E*)w2, \
+                     coef, (const E*)w_post, (const E*)w_next, W, eps)
+  DISPATCH_SEQ_DTYPE(dtype, {
+    typedef typename El<P>::type E;
+    if (W <= 512) PAIR_SEAM(2);
+    else if (W <= 2048) PAIR_SEAM(8);
+    else if (W <= 4096) PAIR_SEAM(16);
+    else PAIR_SEAM(0);
+  })
+#undef PAIR_SEAM
   UMB_LAUNCH_CHECK();
   return UMB_OK;
 }

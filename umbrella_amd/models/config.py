@@ -300,6 +300,27 @@ def rotary_frequencies(base: float, dims: int, scaling: Optional[dict] = None) -
     return f.to(torch.float32)
 
 
+def yarn_frequencies(base: float, dims: int, scaling: dict) -> tuple[torch.Tensor, float]:
+    """(fp32 [dims / 2], factor on cos and sin).  ``scaling`` = {factor, original, fast, slow}: over ``original`` positions the
+    pair i turns original f_i / (2 pi) times, so t turns belong to the pair at index(t) = dims ln(original / (2 pi t)) / (2 ln base).
+    Pairs up to floor(index(fast)) keep f_i, pairs from ceil(index(slow)) on get f_i / factor, a linear ramp in between (YaRN);
+    cos and sin grow by 0.1 ln(factor) + 1.  Formed in float64 and rounded once."""
+    factor, orig = float(scaling["factor"]), float(scaling["original"])
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = float(base) ** (-2.0 * i / dims)
+    index = lambda turns: dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(base))     # noqa: E731
+    lo, hi = max(math.floor(index(float(scaling["fast"]))), 0), min(math.ceil(index(float(scaling["slow"]))), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return (f / factor * ramp + f * (1.0 - ramp)).to(torch.float32), 0.1 * math.log(factor) + 1.0
+
+
+def rotary_table(base: float, dims: int, scaling: Optional[dict] = None) -> tuple[torch.Tensor, float]:
+    """(fp32 frequencies [dims / 2], factor on cos and sin) under either kind of frequency scaling, or none"""
+    if scaling and "fast" in scaling:
+        return yarn_frequencies(base, dims, scaling)
+    return rotary_frequencies(base, dims, scaling), 1.0
+
+
 @dataclass
 class RetentionCfg:
     """Linear attention with one FIXED decay per head (``decay``: a number per head) and neither softmax nor denominator:
@@ -355,8 +376,53 @@ class AttnMLSTMCfg:
 
 
 @dataclass
+class DiffAttnCfg:
+    """Differential attention: every head has two query / key maps over the same values; its output is ``a1 - lambda a2`` (one
+    lambda per layer, from four vectors and the constant ``diff``) over its root mean square, times ``1 - diff``.  Grouped query
+    heads, rotary positions on the first ``rot_dims`` features of every map, keys of the query's own run of ``chunk`` positions
+    only (0: every earlier position).  ``kv_from``: the layer reads that layer's keys and values and has none of its own."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    diff: float
+    chunk: int
+    rot_dims: int
+    rot_base: float
+    rot_scaling: Optional[dict] = None
+    rot_layout: str = "half"
+    kv_from: Optional[int] = None
+    kind: str = "diff_attention"
+
+
+@dataclass
+class AttnDeltaCfg:
+    """Two mixers side by side that read the same input, each with its own output projection; ``pair_coef`` times the sum of the
+    two outputs, each first RMS-normed over the width with a weight of its own, is the mixer's output.
+
+    Attention: causal softmax without positions, grouped query heads, q / k RMS-normed per head (weights shared by the heads), a
+    sink of score 0 in the denominator.
+    Gated delta rule: ``s_heads`` value heads of ``s_vdim`` over ``s_groups`` query / key heads of ``s_state``, an ``[s_state, s_vdim]``
+    fp32 state per value head, one decay and one step size per head, a causal convolution of ``s_taps`` taps in front, a gated
+    per-head RMS norm behind."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    s_heads: int
+    s_groups: int
+    s_state: int
+    s_vdim: int
+    s_taps: int
+    pair_coef: float = 0.5
+    kind: str = "attention_delta"
+
+
+@dataclass
 class SeqLayerCfg:
-    mixer: object                    # PooledWindowAttnCfg | GLACfg | LatentAttnCfg | MinGRUCfg | AttnSSDCfg | RetentionCfg | AttnMLSTMCfg
+    mixer: object                    # one of the mixer descriptions above
     ff: int = 0                      # width of the dense feed-forward; 0 = the layer has none (or has experts)
     ff_kind: str = "gated"           # "gated": W_down (silu(W_gate h) * W_up h); "polynorm": W_down polynorm(W_up h); "moe"
     experts: int = 0                 # "moe": routed experts, how many each token uses, their width, the shared expert's

@@ -1,14 +1,15 @@
 """Runtime of the sequence-mixer model family on the HIP path (libumbrella_seq.so, include/umbrella_seq.h).
 
 A model is a LIST of layers, each a token mixer -- windowed attention with pooled blocks, gated linear attention, latent
-attention, a minimal gated recurrence, softmax attention beside a state-space layer, retention, or convolved softmax
-attention beside a matrix memory -- plus an optional feed-forward (gated SiLU, PolyNorm, or routed experts with a shared one).  A sublayer reads either a grouped RMS norm of the residual stream or the
+attention, a minimal gated recurrence, softmax attention beside a state-space layer, retention, convolved softmax attention
+beside a matrix memory, differential attention (over its own or another layer's keys and values), or attention with a sink
+beside a gated delta rule -- plus an optional feed-forward (gated SiLU, PolyNorm, or routed experts with a shared one).  A sublayer reads either a grouped RMS norm of the residual stream or the
 stream itself through a short causal convolution; its output is normed before it is added back; or (``streams >= 1``) the
 residual is several streams that every sublayer reads as one combination and writes back to all.  A layer may use another
 layer's tensors with a cache and state of its own; or (``block == "parallel"``) both sublayers of a layer read the same
 residual and their outputs are added to it together.  The list, every size and every
 constant come from a ``SeqMixCfg`` (models/config.py); a design contributes a subclass that names its checkpoint tensors
-(models/gitopel.py, models/fidizen.py).
+(models/gitopel.py, fidizen.py, tomopel.py, zusuvik.py, tutunex.py).
 
 Unlike the tree-decoding ``Llama`` runtime this one serves MANY sequences: a step is a ragged batch (the rows of each
 sequence contiguous, nothing padded), key/value pages and recurrent-state slots are handed out by
@@ -28,10 +29,10 @@ from .. import _lib
 from .._lib import UmbSeqLayer, UmbSeqLinear, UmbSeqModel, UmbSeqStep, UmbSeqWork
 from ..attn.cache import PagedSeqCache
 from .base import LLMBase
-from .config import SeqMixCfg, rotary_frequencies
+from .config import SeqMixCfg, rotary_frequencies, rotary_table
 
 KIND_CODE = {"attention": 0, "gla": 1, "latent_attention": 2, "mingru": 3, "attention_ssd": 4, "retention": 5,
-             "attention_mlstm": 6}
+             "attention_mlstm": 6, "diff_attention": 7, "attention_delta": 8}
 FF_CODE = {"gated": 0, "polynorm": 1, "moe": 2}
 ACT_CODE = {"silu_gated": 0, "relu2": 1, "clamp_glu": 2}
 ROUTE_CODE = {"sigmoid_in": 0, "softmax_out": 1, "top_logits": 2}
@@ -156,6 +157,30 @@ class SeqMixLM(LLMBase):
                 state_layers.append((m.m_heads, m.m_dim, m.m_pad))      # value column m_vdim carries the normaliser
                 state_layers.append((m.m_heads, 1, 1))                  # the running maximum
                 mixer_convs.append((m.taps, (m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim))
+            elif m.kind == "diff_attention":
+                if m.heads % m.kv_heads:
+                    raise ValueError("heads must be a multiple of kv_heads")
+                if m.kv_from is None:
+                    t["cache_index"] = len(kv_layers)
+                    kv_layers.append((m.kv_heads, 2 * m.dim, 0, m.vdim))        # a cached key row is [map 1 | map 2]
+                else:                                                          # the store of a layer that has projections of its own
+                    src = c.layers[m.kv_from].mixer if 0 <= m.kv_from < i else None
+                    if src is None or src.kind != m.kind or src.kv_from is not None:
+                        raise ValueError(f"layer {i}: kv_from must name an earlier layer with keys and values of its own")
+                    if (src.kv_heads, src.dim, src.vdim) != (m.kv_heads, m.dim, m.vdim):
+                        raise ValueError(f"layer {i}: kv_from wants equal key / value heads and sizes")
+                    t["cache_index"] = self._tensors[m.kv_from]["cache_index"]
+            elif m.kind == "attention_delta":
+                if m.heads % m.kv_heads or m.s_heads % m.s_groups:
+                    raise ValueError("heads must be a multiple of kv_heads on both sides")
+                if m.s_state > 256:
+                    raise ValueError("the delta rule's kernels cover keys of up to 256 features")
+                t["cache_index"], t["state_index"], t["mconv_index"] = len(kv_layers), len(state_layers), len(mixer_convs)
+                kv_layers.append((m.kv_heads, m.dim, 0, m.vdim))
+                state_layers.append((m.s_heads, m.s_state, m.s_vdim))
+                # one ring row more than the convolution looks back: single-token steps read and refresh it side by side
+                mixer_convs.append((m.s_taps + 1, 2 * m.s_groups * m.s_state + m.s_heads * m.s_vdim))
+                t["attn_sink"] = torch.zeros(m.heads, dtype=torch.float32, device=dev)
             else:
                 t["cache_index"] = len(state_layers)
                 state_layers.append((m.heads, m.dim, m.vdim))
@@ -164,6 +189,9 @@ class SeqMixLM(LLMBase):
                 t["rot_freq"] = (m.rot_base ** (-2 * i2 / m.rot_dims)).to(dev) if m.rot_dims else None     # fp32 frequencies
             if m.kind in ("retention", "attention_mlstm") and "rot_freq" not in t:
                 t["rot_freq"] = rotary_frequencies(m.rot_base, m.rot_dims, m.rot_scaling).to(dev) if m.rot_dims else None
+            if m.kind == "diff_attention":
+                freq, t["rot_mult"] = rotary_table(m.rot_base, m.rot_dims, m.rot_scaling) if m.rot_dims else (None, 1.0)
+                t["rot_freq"] = freq.to(dev) if freq is not None else None
             if c.canon_taps > 0:
                 t["conv_index"] = n_conv
                 n_conv += 2 if ly.has_ff else 1
@@ -238,6 +266,23 @@ class SeqMixLM(LLMBase):
                 s.kv = self.kv_cache.struct(t["cache_index"])
                 s.state = self.kv_cache.state[t["state_index"]].data_ptr()
                 s.m_max = self.kv_cache.state[t["state_index"] + 1].data_ptr()
+            elif m.kind == "diff_attention":
+                s.kv_heads, s.scale, s.window, s.chunk = m.kv_heads, float(m.scale), 2 ** 30, int(m.chunk)
+                s.rot_dims, s.rot_layout, s.rot_mult = m.rot_dims, ROT_LAYOUT_CODE[m.rot_layout], float(t["rot_mult"])
+                s.rot_freq = t["rot_freq"].data_ptr() if t["rot_freq"] is not None else None
+                s.kv_shared, s.diff_lambda, s.out_mult = int(m.kv_from is not None), float(t["diff_lambda"]), 1.0 - float(m.diff)
+                s.kv = self.kv_cache.struct(t["cache_index"])
+            elif m.kind == "attention_delta":
+                s.kv_heads, s.scale, s.window = m.kv_heads, float(m.scale), 2 ** 30
+                s.q_norm, s.k_norm, s.attn_sink = t["q_norm"].data_ptr(), t["k_norm"].data_ptr(), t["attn_sink"].data_ptr()
+                s.s_heads, s.s_groups, s.s_state, s.s_vdim, s.s_taps = m.s_heads, m.s_groups, m.s_state, m.s_vdim, m.s_taps
+                s.s_conv, s.s_norm = t["s_conv"].data_ptr(), t["s_norm"].data_ptr()
+                s.s_dt_bias, s.s_a_log = t["s_dt_bias"].data_ptr(), t["s_a_log"].data_ptr()
+                s.s_conv_state = self.kv_cache.mixer_conv[t["mconv_index"]].data_ptr()
+                s.out2, s.pair_coef = _linear(t["out2_w"]), float(m.pair_coef)
+                s.out_norm_a, s.out_norm_b = t["out_norm_a"].data_ptr(), t["out_norm_b"].data_ptr()
+                s.kv = self.kv_cache.struct(t["cache_index"])
+                s.state = self.kv_cache.state[t["state_index"]].data_ptr()
             else:
                 s.rank, s.tau, s.qscale = m.rank, m.tau, float(m.dim) ** -0.5
                 s.a2, s.head_norm = _linear(t["a2_w"], t["a2_b"]), t["head_norm"].data_ptr()
@@ -316,6 +361,16 @@ class SeqMixLM(LLMBase):
                 conv_row = (m.heads + m.kv_heads) * m.dim + 2 * (((m.heads + m.kv_heads) * m.dim + m.kv_heads * m.vdim + 255) // 256)
                 ask(aux=m.heads * m.dim + max(conv_row, m.m_heads * (m.m_dim + m.m_pad + 5) + (chunk + 63) // 64 + (8 * chunk + 64) // T + 1),
                     o=m.m_heads * m.m_pad, mix=m.heads * m.vdim + m.m_heads * m.m_vdim)
+            elif m.kind == "diff_attention":
+                # aux: queries of both maps, and room for the partial results of split keys (16 a row and more for few rows)
+                ask(aux=2 * m.heads * m.dim + 32 * m.heads * (m.vdim + 2) // (16 if T > 64 else 1) + 4, mix=m.heads * m.vdim)
+            elif m.kind == "attention_delta":
+                # aux: queries | delta-rule q, k, v, step sizes, log decays | the chunk kernels' scratch; mix: the two mixers' rows
+                up = lambda n: (n + 15) // 16 * 16                                                        # noqa: E731
+                inner = m.s_heads * m.s_vdim
+                rows = 2 * m.s_groups * up(m.s_state) + inner + 2 * m.s_heads + m.s_heads * (up(m.s_state) + up(m.s_vdim) + 66)
+                ask(aux=m.heads * m.dim + max(rows, 16 * m.heads * (m.vdim + 2) // (16 if T > 64 else 1)) + 48 // T + 2, o=inner,
+                    mix=m.heads * m.vdim + inner + 64 // T + 1)
             else:
                 ask(aux=m.heads * m.dim, o=m.heads * m.vdim, mix=m.heads * m.vdim)
             if ly.ff_kind == "moe":
@@ -333,9 +388,12 @@ class SeqMixLM(LLMBase):
         ws = self._ws = UmbSeqWork()
         for k in ("x", "h", "proj", "aux", "o", "mix", "act", "y", "logits"):
             setattr(ws, k, b[k].data_ptr())
-        if c.block == "parallel":                       # the feed-forward's own normed input and output
-            b.update(h2=torch.zeros(T, c.width, dtype=dt, device=dev), y2=torch.zeros(T, c.width, dtype=f32, device=dev))
-            ws.h2, ws.y2 = b["h2"].data_ptr(), b["y2"].data_ptr()
+        if c.block == "parallel":                       # the feed-forward's own normed input
+            b["h2"] = torch.zeros(T, c.width, dtype=dt, device=dev)
+            ws.h2 = b["h2"].data_ptr()
+        if c.block == "parallel" or any(ly.mixer.kind == "attention_delta" for ly in c.layers):
+            b["y2"] = torch.zeros(T, c.width, dtype=f32, device=dev)     # its output; the second output projection's
+            ws.y2 = b["y2"].data_ptr()
         if top:
             pairs = T * top
             tiles = (pairs + 15) // 16 + max(ly.experts for ly in c.layers)          # the smallest tile size the forward picks
