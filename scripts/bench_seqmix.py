@@ -20,6 +20,12 @@ synthetic ids.
         beside a state-space layer on the same scans) where Zusuvik has its own, minGRU layers where it has retention, routed
         experts everywhere -- at equal width, heads x head size, state size, expert width and layer count
 
+    python bench.py --family tutunex [--sizes 1b,8b] ...
+        Tutunex (differential attention over chunks, own or another layer's keys and values; sink attention beside a gated delta
+        rule; capped-GLU feed-forwards), whole and kind by kind beside the closest existing layers: its parallel layers beside
+        Tomopel's (attention beside a state-space layer of the same state size, a dense gated feed-forward), its
+        differential layers beside Gitopel's windowed attention (window = chunk), at equal width, head rows and layer count
+
 or directly: python scripts/bench_seqmix.py.  One JSON line: per size, ms and tokens/s of
   prefill   one prompt of --prompt-len tokens in one step (Llama: its chunked prompt path)
   decode    one token per step behind that prompt, batch 1 (both) and batch --batch (Gitopel; the Llama runtime is batch 1)
@@ -79,6 +85,38 @@ ZUS_SIZES = {
 }
 
 
+# Tutunex: "p" layers are attention (heads x dim over kv_heads) beside a delta rule (s_heads x s_vdim values over s_groups x state
+# keys), "d" layers differential attention (d_heads of two maps of d_dim, values d_vdim, over d_kv), "s" layers the same over the
+# keys and values of the last "d" layer
+TUT_SIZES = {
+    "1b": dict(width=2048, ff=8192, heads=32, kv_heads=8, dim=64, vdim=64, s_heads=16, s_groups=8, s_vdim=128, state=128, conv=4,
+               d_heads=16, d_kv=4, d_dim=64, d_vdim=128, chunk=1024, pattern="pdsp", vocab=32000),
+    "8b": dict(width=4096, ff=14336, heads=32, kv_heads=8, dim=128, vdim=128, s_heads=32, s_groups=16, s_vdim=128, state=128, conv=4,
+               d_heads=16, d_kv=4, d_dim=128, d_vdim=256, chunk=1024, pattern="pds", vocab=32000),
+}
+
+
+def tutunex_config(s):
+    layers, last = [], None
+    for i, ch in enumerate(s["pattern"]):
+        mlp = {"kind": "dense", "ff": s["ff"], "limit": 7.0}
+        if ch == "p":
+            mixer = {"left": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": s["dim"], "vdim": s["vdim"], "scale": s["dim"] ** -0.5},
+                     "right": {"heads": s["s_heads"], "kv_heads": s["s_groups"], "dim": s["state"], "vdim": s["s_vdim"], "conv": s["conv"]}}
+            layers.append({"type": "parallel", "mixer": mixer, "mlp": mlp})
+        else:
+            mixer = {"heads": s["d_heads"], "kv_heads": s["d_kv"], "dim": s["d_dim"], "vdim": s["d_vdim"], "diff": 0.5,
+                     "scale": s["d_dim"] ** -0.5, "mask": {"size": s["chunk"]},
+                     "rot": {"base": 500000.0, "dims": s["d_dim"], "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+            if ch == "s":
+                mixer["kv_from"] = last
+            else:
+                last = i
+            layers.append({"type": "attention", "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Tutunex", "layers": layers, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "vocab": s["vocab"],
+            "width": s["width"]}
+
+
 def zusuvik_config(s):
     layers = []
     mlp = {"kind": "moe", "router": {"experts": s["experts"], "top": s["top"]}, "expert": {"ff": s["ff"] // 4, "limit": 7.0},
@@ -110,7 +148,7 @@ def tomopel_config(s):
             kind = "parallel"
         else:
             mixer, kind = {"width": s["width"]}, "mingru"
-        if i % 2 == 0 and not s.get("all_moe"):
+        if s.get("all_dense") or (i % 2 == 0 and not s.get("all_moe")):
             mlp = {"kind": "dense", "ff": s["ff"]}
         else:
             mlp = {"kind": "moe", "router": {"experts": s["experts"], "top": s["top"]}, "expert": {"ff": s["ff"] // 4},
@@ -178,15 +216,19 @@ def timed(fn, reps):
     return (time.time() - t0) / reps * 1e3
 
 
-def bench_gitopel(s, args, dtype, fidizen=False, tomopel=False, zusuvik=False):
+def bench_gitopel(s, args, dtype, fidizen=False, tomopel=False, zusuvik=False, tutunex=False):
     from umbrella_amd.models import fidizen as fid
     from umbrella_amd.models import gitopel
     from umbrella_amd.models import tomopel as tom
+    from umbrella_amd.models import tutunex as tut
     from umbrella_amd.models import zusuvik as zus
     B, P, steps = args.batch, args.prompt_len, args.decode_steps
     kw = dict(batch_size=B + 1, max_length=P + 2 * steps + 8, max_tokens=(B + 1) * (P + 2 * steps + 8), device="cuda:0",
               dtype=dtype, max_step_tokens=max(P, B))
-    if zusuvik:
+    if tutunex:
+        cfg = tut.config_from_dict(tutunex_config(s))
+        m = tut.Tutunex("bench", state_dict=device_state(cfg, dtype, shapes=tut.tensor_shapes(cfg)), config=cfg, **kw)
+    elif zusuvik:
         cfg = zus.config_from_dict(zusuvik_config(s))
         sd = device_state(cfg, dtype, shapes=zus.tensor_shapes(cfg), zero_norms=True)
         m = zus.Zusuvik("bench", state_dict=sd, config=cfg, **kw)
@@ -330,6 +372,40 @@ def run_zusuvik(args):
     return line
 
 
+def run_tutunex(args):
+    """Tutunex as a whole, then its two kinds of layers beside the closest existing ones at equal size: parallel layers beside
+    Tomopel's parallel layers, differential attention beside Gitopel's windowed attention"""
+    import __graft_entry__ as ge
+    ge.build_seq()
+    dtype = torch.bfloat16
+    res = {}
+    for name in args.sizes.split(","):
+        s = TUT_SIZES[name]
+        r = res[name] = {"shape": dict(s)}
+        r["tutunex"] = bench_gitopel(s, args, dtype, tutunex=True)
+        torch.cuda.empty_cache()
+        if args.no_gitopel:
+            continue
+        r["tutunex_parallel_layers"] = bench_gitopel(dict(s, pattern="pp"), args, dtype, tutunex=True)
+        torch.cuda.empty_cache()
+        t = dict(width=s["width"], ff=s["ff"], heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], vdim=s["vdim"],
+                 s_heads=s["s_heads"] * s["s_vdim"] // 64, s_vdim=64, state=s["state"], groups=s["s_groups"], conv=s["conv"], experts=8,
+                 top=2, pattern="pp", vocab=s["vocab"], bias_rows=32, bias_max=2048, all_dense=True)
+        r["tomopel_parallel_layers_equal_size"] = bench_gitopel(t, args, dtype, tomopel=True)
+        torch.cuda.empty_cache()
+        r["tutunex_differential_layers"] = bench_gitopel(dict(s, pattern="dd"), args, dtype, tutunex=True)
+        torch.cuda.empty_cache()
+        g = dict(width=s["width"], ff=s["ff"], heads=2 * s["d_heads"], kv_heads=2 * s["d_kv"], dim=s["d_dim"], window=s["chunk"], pool=16,
+                 pattern="aa", vocab=s["vocab"])
+        r["gitopel_attention_layers_equal_size"] = bench_gitopel(g, args, dtype)
+        torch.cuda.empty_cache()
+    line = {"metric": "prefill / decode throughput, Tutunex whole and kind by kind beside the closest layers at equal size",
+            "unit": "tokens/s", "dtype": "bf16", "data": "synthetic: random weights, random ids", "n_gpus": 1,
+            "prompt_len": args.prompt_len, "decode_steps": args.decode_steps, "batch": args.batch, "sizes": res}
+    print(json.dumps(line), flush=True)
+    return line
+
+
 def run(args):
     import __graft_entry__ as ge
     ge.build()
@@ -362,7 +438,7 @@ def add_args(ap):
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--prompt-len", type=int, default=2048)
-    ap.add_argument("--family", default="gitopel", choices=["gitopel", "fidizen", "tomopel", "zusuvik"])
+    ap.add_argument("--family", default="gitopel", choices=["gitopel", "fidizen", "tomopel", "zusuvik", "tutunex"])
     add_args(ap)
     a = ap.parse_args()
-    {"fidizen": run_fidizen, "tomopel": run_tomopel, "zusuvik": run_zusuvik}.get(a.family, run)(a)
+    {"fidizen": run_fidizen, "tomopel": run_tomopel, "zusuvik": run_zusuvik, "tutunex": run_tutunex}.get(a.family, run)(a)
