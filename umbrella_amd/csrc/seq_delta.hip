@@ -14,6 +14,7 @@
 //   delta_chunk_* longer steps: the recurrence in chunks of 64 tokens (below)
 // Everything is fp32.  The convolution sums its taps oldest first whatever their source.
 #include "seq_common.h"
+#include <type_traits>
 
 constexpr float DELTA_UNIT_EPS = 1e-6f;
 
@@ -184,8 +185,8 @@ constexpr int DC_Q = 64;
 
 struct DeltaChunk {
   const float *q, *k, *v, *beta, *lg;      // q, k [T][ldqk] groups of Dp (zero padded from D); v [T][H E]; beta, lg [T][H]
-  float *wk, *uv, *m, *ec, *ew;            // [T][H Dp], [T][H Ep], [T][H 64], [T][H] e^(c_t), [T][H] e^(c_end - c_t)
-  int ldqk, Hk, H, D, Dp, E, Ep;
+  float *wk, *uv, *m, *ec, *ew;            // [T][H Dp], [T][H Ep], [T][H 64], [H][T] e^(c_t), [H][T] e^(c_end - c_t)
+  int T, ldqk, Hk, H, D, Dp, E, Ep;
   const int *seq_slot, *seq_row0, *seq_pos0, *seq_len;
 };
 
@@ -222,8 +223,8 @@ __global__ __launch_bounds__(256) void delta_chunk_solve_kernel(DeltaChunk a) {
     const float e = expf((float)v), w = expf((float)(__shfl(v, 63, 64) - v));
     ecs[lane] = e;
     if (lane < cnt) {
-      a.ec[(row0 + lane) * H + h] = e;
-      a.ew[(row0 + lane) * H + h] = w;
+      a.ec[(long)h * a.T + row0 + lane] = e;
+      a.ew[(long)h * a.T + row0 + lane] = w;
     }
   }
   const int dq = Dp >> 2;
@@ -317,7 +318,8 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(float* __restrict
   const int b = blockIdx.z, h = blockIdx.y, H = a.H, Dp = a.Dp, D = a.D, E = a.E;
   const int n = a.seq_len[b];
   if (n <= 0) return;
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, j = lane & 15, g = lane >> 4, hk = h / (H / a.Hk);
+  const int tid = threadIdx.x, lane = tid & 63, j = lane & 15, g = lane >> 4, hk = h / (H / a.Hk);
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);         // uniform: what depends on it stays in scalar registers
   const int col = blockIdx.x * 16 + j;
   const bool c_ok = col < E;
   const long row0 = a.seq_row0[b];
@@ -333,42 +335,56 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(float* __restrict
     }
   const f32x4 zero = f32x4{0.f, 0.f, 0.f, 0.f};
   const int nch = (n + DC_Q - 1) / DC_Q;
+  const int ldw = H * Dp, ldu = H * a.Ep, ldm = H * 64, ldk = a.ldqk;
+  // The operands of a chunk.  Every load is unconditional: a row past the stretch reads the last row instead, and what it brings
+  // has no effect -- its weight ew is 0, M is 0 above the diagonal, its read-out is not stored.  In a full chunk the row of lane
+  // (j, g) is its lane part plus a uniform part, so an address is a scalar base and one of a few lane offsets.
   auto load = [&](int ch, DeltaFrag<TPW>& f) {
     const int cnt = n - ch * DC_Q < DC_Q ? n - ch * DC_Q : DC_Q;
     const long base = row0 + (long)ch * DC_Q;
+    const float* wk = a.wk + base * ldw + (long)h * Dp + 16 * wave * TPW;
+    const float* q = a.q + base * ldk + (long)hk * Dp + 16 * wave * TPW;
+    const float* k = a.k + base * ldk + (long)hk * Dp + 16 * wave * TPW;
+    const float* uv = a.uv + base * ldu + (long)h * a.Ep + blockIdx.x * 16;
+    const float* m = a.m + base * ldm + (long)h * 64;
+    const float* ec = a.ec + (long)h * a.T + base;
+    const float* ew = a.ew + (long)h * a.T + base;
+    auto fill = [&](auto full) {
+      // row of an operand whose lanes run over rows (u + j) / over groups of four rows (u + 4 g + r): uniform and lane part
+      auto at_j = [&](const float* p, int ld, int u) {
+        return full ? p + u * ld + (unsigned)(j * ld) : p + (unsigned)((u + j < cnt ? u + j : cnt - 1) * ld);
+      };
+      auto at_g = [&](const float* p, int ld, int u) {
+        return full ? p + u * ld + (unsigned)(4 * g * ld) : p + (unsigned)((u + 4 * g < cnt ? u + 4 * g : cnt - 1) * ld);
+      };
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const bool ok = 16 * i + j < cnt;
-      const long row = base + (ok ? 16 * i + j : 0);
-#pragma unroll
-      for (int x = 0; x < TPW; ++x) {
-        const int d = 16 * (wave * TPW + x);
-        const bool in = ok && d < Dp;
-        f.wk[i][x] = in ? *reinterpret_cast<const f32x4*>(a.wk + (row * H + h) * Dp + d + 4 * g) : zero;
-        f.q[i][x] = in ? *reinterpret_cast<const f32x4*>(a.q + row * a.ldqk + (long)hk * Dp + d + 4 * g) : zero;
-      }
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = 16 * i + 4 * g + r;
-        const bool tok = t < cnt;
-        const long tr = base + (tok ? t : 0);
-        f.uv[i][r] = tok ? a.uv[(tr * H + h) * a.Ep + col] : 0.f;
-        f.ew[i][r] = tok ? a.ew[tr * H + h] : 0.f;
+      for (int i = 0; i < 4; ++i) {
 #pragma unroll
         for (int x = 0; x < TPW; ++x) {
-          const int d = 16 * (wave * TPW + x) + j;
-          f.kt[i][x][r] = (tok && d < Dp) ? a.k[tr * a.ldqk + (long)hk * Dp + d] : 0.f;
-        }
-      }
-      const bool mok = i <= wave && 16 * wave + j < cnt;
-      f.m[i] = mok ? *reinterpret_cast<const f32x4*>(a.m + ((base + 16 * wave + j) * H + h) * 64 + 16 * i + 4 * g) : zero;
-    }
+          if (16 * (wave * TPW + x) < Dp) {                          // uniform
+            f.wk[i][x] = *reinterpret_cast<const f32x4*>(at_j(wk + 16 * x, ldw, 16 * i) + 4 * g);
+            f.q[i][x] = *reinterpret_cast<const f32x4*>(at_j(q + 16 * x, ldk, 16 * i) + 4 * g);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = 16 * wave + 4 * g + r;
-      f.ec[r] = t < cnt ? a.ec[(base + t) * H + h] : 0.f;
-    }
-    f.eq = a.ec[(base + cnt - 1) * H + h];
+            for (int r = 0; r < 4; ++r) f.kt[i][x][r] = at_g(k + 16 * x, ldk, 16 * i + r)[j];
+          } else {
+            f.wk[i][x] = f.q[i][x] = f.kt[i][x] = zero;
+          }
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          f.uv[i][r] = at_g(uv, ldu, 16 * i + r)[j];
+          f.ew[i][r] = at_g(ew, 1, 16 * i + r)[0];
+          if (!full && 16 * i + 4 * g + r >= cnt) f.ew[i][r] = 0.f;
+        }
+        if (i <= wave) f.m[i] = *reinterpret_cast<const f32x4*>(at_j(m + 16 * i, ldm, 16 * wave) + 4 * g);
+        else f.m[i] = zero;
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) f.ec[r] = at_g(ec, 1, 16 * wave + r)[0];
+    };
+    if (cnt == DC_Q) fill(std::true_type{});
+    else fill(std::false_type{});
+    f.eq = ec[cnt - 1];
   };
   auto compute = [&](int ch, const DeltaFrag<TPW>& f) {
     const int cnt = n - ch * DC_Q < DC_Q ? n - ch * DC_Q : DC_Q;
@@ -394,7 +410,8 @@ __global__ __launch_bounds__(256) void delta_chunk_scan_kernel(float* __restrict
     for (int w = 0; w < 4; ++w) out += *reinterpret_cast<const f32x4*>(rb + (w * 8 + 4 + wave) * 256 + lane * 4);
     out *= f.ec;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) out = mma4(f.m[i], U[i], out);       // zero above the diagonal
+    for (int i = 0; i < 4; ++i)
+      if (i <= wave) out = mma4(f.m[i], U[i], out);
 #pragma unroll
     for (int x = 0; x < TPW; ++x) S[x] *= f.eq;
 #pragma unroll
@@ -506,7 +523,7 @@ extern "C" int umb_delta_scan(float* o, float* state, const float* q, const floa
   float* m = wk + n * Dp;
   float* uv = m + n * 64;
   float* ec = uv + n * Ep;
-  DeltaChunk a{q, k, v, beta, log_g, wk, uv, m, ec, ec + n, ldqk, Hk, H, D, Dp, E, Ep, seq_slot, seq_row0, seq_pos0, seq_len};
+  DeltaChunk a{q, k, v, beta, log_g, wk, uv, m, ec, ec + n, T, ldqk, Hk, H, D, Dp, E, Ep, seq_slot, seq_row0, seq_pos0, seq_len};
   const size_t lds1 = delta_solve_lds(Dp), lds2 = (size_t)2 * 4 * 8 * 256 * sizeof(float);
   if (ensure_dynamic_lds<delta_chunk_solve_kernel>(lds1) != UMB_OK) return UMB_EHIP;
   hipLaunchKernelGGL(delta_chunk_solve_kernel, dim3((max_len + DC_Q - 1) / DC_Q, H, B), dim3(256), lds1, st, a);
