@@ -4,7 +4,9 @@
  * libumbrella_hip.so: gated linear attention (a per-head matrix state carried from token to token) and sliding-window
  * attention over a paged key/value store with mean-pooled blocks behind the window and sigmoid (un-normalised) weights;
  * latent attention; a minimal gated recurrence; softmax attention with a bias by distance beside a state-space layer with a
- * scalar decay per head; differential attention over chunks of positions; attention with a sink beside a gated delta rule; residuals of one or several streams; dense, PolyNorm and routed-expert feed-forwards.
+ * scalar decay per head; differential attention over chunks of positions; attention with a sink beside a gated delta rule; softmax
+ * attention by form (window with kept first tokens or chunks, bias by distance, rotary, sink, gate, values mixed over layers); residuals
+ * of one or several streams; dense, PolyNorm and routed-expert feed-forwards.
  * The layer list, every size and every constant are data (UmbSeqLayer); one forward entry point walks the list.
  *
  * Conventions are those of umbrella_hip.h: extern "C", plain pointers and sizes, 0 or a negative errno-style code,
@@ -29,12 +31,14 @@ typedef struct ihipStream_t* umb_stream_t;   /* == hipStream_t */
 
 enum { UMB_SEQ_F16 = 0, UMB_SEQ_BF16 = 1, UMB_SEQ_F32 = 2 };
 enum { UMB_MIX_POOLED_WINDOW = 0, UMB_MIX_GLA = 1, UMB_MIX_LATENT = 2, UMB_MIX_MINGRU = 3, UMB_MIX_ATTN_SSD = 4,
-       UMB_MIX_RETENTION = 5, UMB_MIX_ATTN_MLSTM = 6, UMB_MIX_DIFF_ATTN = 7, UMB_MIX_ATTN_DELTA = 8 };
+       UMB_MIX_RETENTION = 5, UMB_MIX_ATTN_MLSTM = 6, UMB_MIX_DIFF_ATTN = 7, UMB_MIX_ATTN_DELTA = 8,
+       UMB_MIX_SOFTMAX = 9 };
 /* feed-forward kinds: gated SiLU (W_down (silu(W_gate h) * W_up h)), PolyNorm (W_down polynorm(W_up h)), routed experts */
 enum { UMB_FF_GATED = 0, UMB_FF_POLYNORM = 1, UMB_FF_MOE = 2 };
-/* activation of a feed-forward / expert: silu(W_gate h) * (W_up h) over stacked [gate; up], relu(W_up h)^2 (no gate), or the
- * capped form g sigmoid(alpha g) (u + 1) with g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit) over stacked [gate; up] */
-enum { UMB_ACT_SILU_GATED = 0, UMB_ACT_RELU2 = 1, UMB_ACT_CLAMP_GLU = 2 };
+/* activation of a feed-forward / expert: silu(W_gate h) * (W_up h) over stacked [gate; up], relu(W_up h)^2 (no gate), the
+ * capped form g sigmoid(alpha g) (u + 1) with g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit) over stacked [gate; up], or
+ * gelu(W_gate h) * (W_up h) with the tanh form of gelu */
+enum { UMB_ACT_SILU_GATED = 0, UMB_ACT_RELU2 = 1, UMB_ACT_CLAMP_GLU = 2, UMB_ACT_GELU_GATED = 3 };
 /* routing of experts: sigmoid scores that multiply the expert's input; or softmax scores, chosen with a correction added,
  * renormalised over the chosen ones, that multiply the expert's output */
 enum { UMB_ROUTE_SIGMOID_IN = 0, UMB_ROUTE_SOFTMAX_OUT = 1, UMB_ROUTE_TOP_LOGITS = 2 };
@@ -51,13 +55,14 @@ typedef struct UmbSeqLinear { const void* w; const void* bias; int32_t N, K; } U
 
 /* out[T][N] = x[T][K] . W^T + bias, fp32 accumulation in a fixed order that depends on (N, K) only.
  * epi 0: out fp32; epi 1: out in `dtype`; epi 2: W stacks [gate; up] (N = 2 N'), out[T][N'] in `dtype` =
- * silu(gate) * up; epi 4: out in `dtype` = relu(acc)^2.  x and W in `dtype`. */
+ * silu(gate) * up; epi 4: out in `dtype` = relu(acc)^2; epi 6: as 2 with gelu (tanh form).  x and W in `dtype`. */
 int umb_seq_linear(void* out, const void* x, const void* w, const void* bias, int T, int N, int K, int epi, int dtype,
                    umb_stream_t stream);
 
 /* The same product for `batch` independent problems (blockIdx.z): problem b reads x + b sx (rows ldx apart), weights
  * w + b sw ([N][K]) and writes out + b so (rows ldo apart); strides in elements; no bias.  epi 0 / 1 as above;
- * epi 3: out in `dtype` = acc * sigmoid(gate[t ldg + b sg + n]) (gate fp32).  The K order of an output is that of
+ * epi 3: out in `dtype` = acc * sigmoid(gate[t ldg + b sg + n]) (gate fp32); epi 7: the same with ONE gate per row and problem,
+ * gate[t ldg + b sg].  The K order of an output is that of
  * umb_seq_linear. */
 int umb_seq_linear_batched(void* out, const void* x, const void* w, int T, int N, int K, int ldx, int ldo, int batch, long sx,
                            long sw, long so, int epi, const float* gate, int ldg, int sg, int dtype, umb_stream_t stream);
@@ -67,6 +72,10 @@ int umb_seq_linear_batched(void* out, const void* x, const void* w, int T, int N
  * group); 128: both operands staged through LDS (16-bit storage, K and gs multiples of 8). */
 int umb_seq_linear_grouped(void* out, const void* x, const void* w, const int* tiles, int max_tiles, int tile_rows, long gs,
                            int N, int K, int epi, int dtype, umb_stream_t stream);
+
+/* out fp32 [T][N] = cap tanh((x . W^T + bias) / cap): a product whose results are capped (logits) */
+int umb_seq_linear_cap(void* out, const void* x, const void* w, const void* bias, int T, int N, int K, float cap, int dtype,
+                       umb_stream_t stream);
 
 /* RMS norm in `groups` equal consecutive parts of a row: part / sqrt(mean(part^2) + eps), whole row times w.
  * x fp32 [*][W]; rows: optional gather (row i of out comes from row rows[i] of x); out_f32 and/or out_dt may be given. */
@@ -186,6 +195,12 @@ int umb_lat_prep(void* cq, const UmbPagedKV* kv, const float* proj, int ld, cons
  * batched product with W_uk^T) */
 int umb_lat_qsplit(void* qn, float* qa, const float* q, const int* pos, const float* freq, int T, int H, int D, int R,
                    int kv_rank, int rot_dims, int dtype, umb_stream_t stream);
+/* Queries straight from the input projection (no latent of theirs), all of the above in one launch: proj columns q_col.. = the
+ * queries head by head [unrotated D | rotated R], kv_col.. = [latent kv_rank | rotated key part R].  qn, qa and the cache row as above;
+ * layout 0 pairs feature i with i + rot_dims / 2, 1 pairs 2i with 2i + 1; cos and sin times rot_mult. */
+int umb_lat_front(void* qn, float* qa, const UmbPagedKV* kv, const float* proj, int ld, int q_col, int kv_col, const void* w_kv,
+                  const int* pos, const int* slot, const float* freq, int T, int H, int D, int R, int kv_rank, int rot_dims, int layout,
+                  float rot_mult, float eps, int dtype, umb_stream_t stream);
 /* softmax attention of qa over the cached rows of the window (0 <= i - j < window) with a sink per head in the
  * denominator (exp(sink[h]): no key, no value, not scaled; sink may be null); out [T][H][kv_rank] in `dtype`. */
 int umb_lat_attend(void* out, const float* qa, const UmbPagedKV* kv, const void* sink, const int* pos, const int* slot, int T,
@@ -284,15 +299,24 @@ int umb_bsa_attend_tiled(void* out, int ldo, const float* q, const UmbPagedKV* k
 /* ---- the same attention in its general form.  UmbAttnForm: maps 2: differential attention (every head has two query / key maps
  * over the same values: q [T][H][2][D], cached key rows [map 1 | map 2] of 2 D; a head's output is a1 - lambda a2 over its root
  * mean square (eps), times out_scale and the gate); chunk > 0: position i sees only keys of its own run of `chunk` positions
- * counted from position 0; sink fp32 [H] (null: none): exp(sink[h]) joins the softmax denominator.
+ * counted from position 0; sink fp32 [H] (null: none): exp(sink[h]) joins the softmax denominator; keep_first: the first keep_first
+ * positions are visible to every later position whatever window and chunk hide, at their true distance; gate_elem: the gate is H E
+ * columns, output element h E + d times sigmoid(gate[t][h E + d]).
  * prep: columns [q (H maps D) | k (G maps D) | v (G E)] of proj, with append 0 [q] alone (the keys and values are another layer's);
  * norm_qk / norm_v: unit RMS per head (and map), w_q / w_k [D] null: 1; then rotary positions on the first rot_dims features of
  * every map (layout 0: i with i + rot_dims / 2, 1: 2i with 2i + 1; cos and sin times rot_mult); query temperature as above.
  * umb_bsa_prep / umb_bsa_attend / umb_bsa_attend_tiled are the cases without a form. */
-typedef struct UmbAttnForm { int32_t maps, chunk; const float* sink; float lambda, eps; } UmbAttnForm;
+typedef struct UmbAttnForm { int32_t maps, chunk; const float* sink; float lambda, eps; int32_t keep_first, gate_elem; } UmbAttnForm;
+/* values mixed over layers, fp32 rows [T][G E] of the same tokens: first (null: none) = an earlier layer's values, what is cached is
+ * (1 - lambda) v + lambda first; keep (null: none) = where this layer's own v go */
+typedef struct UmbValueMix { const float* first; float* keep; float lambda, pad_; } UmbValueMix;
 int umb_attn_prep(float* q, const UmbPagedKV* kv, const float* proj, int ld, int append, const void* w_q, const void* w_k, int norm_qk,
                   int norm_v, const int* pos, const int* slot, const float* freq, int rot_dims, int layout, float rot_mult, int T,
                   int H, int G, int D, int E, int maps, float temp_coef, int temp_every, float eps, int dtype, umb_stream_t stream);
+int umb_attn_prep_mix(float* q, const UmbPagedKV* kv, const float* proj, int ld, int append, const void* w_q, const void* w_k, int norm_qk,
+                      int norm_v, const int* pos, const int* slot, const float* freq, int rot_dims, int layout, float rot_mult, int T,
+                      int H, int G, int D, int E, int maps, float temp_coef, int temp_every, float eps, const UmbValueMix* mix, int dtype,
+                      umb_stream_t stream);
 int umb_attn_attend(void* out, int ldo, const float* q, const UmbPagedKV* kv, const float* proj, int ld, int gate_col,
                     const float* bias, int n_dist, const int* pos, const int* slot, int T, int H, int G, int D, int E, int window,
                     float scale, float out_scale, float softcap, const UmbAttnForm* form, float* scratch, long scratch_floats,
@@ -487,6 +511,14 @@ typedef struct UmbSeqLayer {
   const float* attn_sink;
   UmbSeqLinear out2;
   const void *out_norm_a, *out_norm_b;
+  /* softmax attention by form (kind 9): proj = [q (heads dim) | k (kv_heads dim) | v (kv_heads vdim) | gate (heads vdim, where gate_elem)];
+   * q_norm / k_norm [dim] (null: no norm), rotary as above (rot_dims 0: none), scale, window with keep_first, chunk, dist_bias / n_dist
+   * (null: none), attn_sink (null: none); v_mix 0: values as projected, 1: the same and kept for later layers of the step (ws.v_first),
+   * 2: mixed with the kept ones, (1 - v_lambda) v + v_lambda v_first.
+   * latent attention with q_rank 0: proj = [q (heads (dim + rot_dim)) | dkv | gate], rotation by rot_layout / rot_mult; gate_head: the
+   * gate is one column per head */
+  int32_t keep_first, gate_elem, gate_head, v_mix;
+  float v_lambda, pad5_;
 } UmbSeqLayer;
 
 typedef struct UmbSeqModel {
@@ -499,7 +531,7 @@ typedef struct UmbSeqModel {
    * the norm of the sum of the streams; 0: the single-stream forms above */
   int32_t streams, block;    /* block: UMB_BLOCK_* (parallel: norms stored around norm_offset, ws.h2 / ws.y2 in use) */
   float resid_mult, norm_offset;
-  float logit_scale, pad2_;  /* the logits are multiplied by it (0 or 1: as they are) */
+  float logit_scale, logit_cap;  /* the logits are multiplied by it (0 or 1: as they are); then cap tanh(logits / cap) (0: not) */
 } UmbSeqModel;
 
 /* activations of one step (caller-owned, sized for Tmax rows) */
@@ -526,6 +558,7 @@ typedef struct UmbSeqWork {
   int64_t aux_floats;  /* floats in aux (what a step does not use of it serves as scratch) */
   void* h2;            /* parallel blocks: normed input of the feed-forward [Tmax][W] dtype */
   float* y2;           /* parallel blocks: feed-forward output; mixers with two output projections: the second [Tmax][W] fp32 */
+  float* v_first;      /* values that later layers of the step mix in [Tmax][kv_heads vdim] fp32 (null when no layer does) */
 } UmbSeqWork;
 
 typedef struct UmbSeqStep {

@@ -244,11 +244,18 @@ class UmbSeqLayer(C.Structure):
                 ("add_embed", C.c_int32), ("pad4_", C.c_int32),
                 ("chunk", C.c_int32), ("kv_shared", C.c_int32), ("rot_mult", C.c_float), ("diff_lambda", C.c_float),
                 ("out_mult", C.c_float), ("pair_coef", C.c_float), ("attn_sink", C.c_void_p), ("out2", UmbSeqLinear),
-                ("out_norm_a", C.c_void_p), ("out_norm_b", C.c_void_p)]
+                ("out_norm_a", C.c_void_p), ("out_norm_b", C.c_void_p),
+                ("keep_first", C.c_int32), ("gate_elem", C.c_int32), ("gate_head", C.c_int32), ("v_mix", C.c_int32),
+                ("v_lambda", C.c_float), ("pad5_", C.c_float)]
 
 
 class UmbAttnForm(C.Structure):
-    _fields_ = [("maps", C.c_int32), ("chunk", C.c_int32), ("sink", C.c_void_p), ("lambda_", C.c_float), ("eps", C.c_float)]
+    _fields_ = [("maps", C.c_int32), ("chunk", C.c_int32), ("sink", C.c_void_p), ("lambda_", C.c_float), ("eps", C.c_float),
+                ("keep_first", C.c_int32), ("gate_elem", C.c_int32)]
+
+
+class UmbValueMix(C.Structure):
+    _fields_ = [("first", C.c_void_p), ("keep", C.c_void_p), ("lambda_", C.c_float), ("pad_", C.c_float)]
 
 
 class UmbSeqModel(C.Structure):
@@ -256,7 +263,7 @@ class UmbSeqModel(C.Structure):
                 ("canon_taps", C.c_int32), ("eps", C.c_float), ("embed_scale", C.c_float), ("embed", C.c_void_p),
                 ("final_norm", C.c_void_p), ("head", UmbSeqLinear), ("layers", C.POINTER(UmbSeqLayer)),
                 ("streams", C.c_int32), ("block", C.c_int32), ("resid_mult", C.c_float), ("norm_offset", C.c_float),
-                ("logit_scale", C.c_float), ("pad2_", C.c_float)]
+                ("logit_scale", C.c_float), ("logit_cap", C.c_float)]
 
 
 class UmbSeqWork(C.Structure):
@@ -265,7 +272,7 @@ class UmbSeqWork(C.Structure):
                 ("Tmax", C.c_int32), ("Rmax", C.c_int32), ("moe_sel", C.c_void_p), ("moe_wt", C.c_void_p),
                 ("moe_pos", C.c_void_p), ("moe_tiles", C.c_void_p), ("moe_xs", C.c_void_p), ("moe_act", C.c_void_p),
                 ("moe_y", C.c_void_p), ("moe_max_tiles", C.c_int64), ("aux_floats", C.c_int64),
-                ("h2", C.c_void_p), ("y2", C.c_void_p)]
+                ("h2", C.c_void_p), ("y2", C.c_void_p), ("v_first", C.c_void_p)]
 
 
 class UmbSeqStep(C.Structure):
@@ -294,6 +301,7 @@ SEQ_SIGNATURES = {
     "umb_moe_combine": [_P, _P, _P, _I, _I, _I, _I],
     "umb_lat_prep": [_P, _PKV, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I],
     "umb_lat_qsplit": [_P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I],
+    "umb_lat_front": [_P, _P, _PKV, _P, _I, _I, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I],
     "umb_lat_attend": [_P, _P, _PKV, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I],
     "umb_lat_attend_tiled": [_P, _P, _PKV, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I],
     "umb_lat_attend_tiled_ok": [_I, _I, _I, _I],
@@ -322,6 +330,7 @@ SEQ_SIGNATURES = {
     "umb_bsa_attend": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P, _L, _I],
     "umb_bsa_attend_tiled": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _I],
     "umb_attn_prep": [_P, _PKV, _P, _I, _I, _P, _P, _I, _I, _P, _P, _P, _I, _I, _F, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I],
+    "umb_attn_prep_mix": [_P, _PKV, _P, _I, _I, _P, _P, _I, _I, _P, _P, _P, _I, _I, _F, _I, _I, _I, _I, _I, _I, _F, _I, _F, _P, _I],
     "umb_attn_attend": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _F, _FORM, _P, _L, _I],
     "umb_attn_attend_tiled": [_P, _I, _P, _PKV, _P, _I, _I, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _FORM, _I],
     "umb_seq_pair_resid_norm": [_P, _P, _P, _P, _P, _P, _F, _P, _P, _I, _I, _F, _I],
@@ -330,6 +339,7 @@ SEQ_SIGNATURES = {
     "umb_delta_scan_floats": [_I, _I, _I, _I],
     "umb_delta_scan": [_P, _P, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _L],
     "umb_seq_linear_glu": [_P, _P, _P, _P, _I, _I, _I, _F, _F, _I],
+    "umb_seq_linear_cap": [_P, _P, _P, _P, _I, _I, _I, _F, _I],
     "umb_seq_linear_grouped_glu": [_P, _P, _P, _P, _I, _I, _L, _I, _I, _F, _F, _I],
     "umb_blk_seam": [_P, _P, _P, _P, _P, _P, _P, _I, _F, _P, _P, _F, _I, _I, _I, _F, _I],
     "umb_seq_scale": [_P, _L, _F],

@@ -13,8 +13,12 @@
 //   maps    2: differential attention -- every head has two query / key maps over the SAME values (a cached key row is [map 1 |
 //           map 2]); with a1, a2 their softmax outputs o = a1 - lambda a2, and the head's o over its root mean square goes out.
 //           The two maps of a head are two rows of one workgroup: the value rows are read once for both.
-// and its prep adds rotary positions (either pair layout, a constant on cos and sin), norms by choice, and queries alone (a
-// layer that reads another layer's keys and values).
+//   keep_first   the first keep_first positions stay visible (at their true distance) whatever the window and the chunk hide:
+//           the walk over the keys takes those of them that lie before its first position in front, as one range
+//   gate_elem    the output gate is a row of H E columns, one sigmoid per output element, instead of one per head
+// and its prep adds rotary positions (either pair layout, a constant on cos and sin), norms by choice, queries alone (a
+// layer that reads another layer's keys and values), and values mixed with those of another layer (UmbValueMix): what is cached is
+// (1 - lambda) v + lambda first, with `first` the same tokens' values as an earlier layer's prep left them.
 //
 // prep: one wave per (token, head slot): query heads -> fp32 q, key heads -> cache K, value heads -> cache V.
 // attend (vector pipe, any dtype and head size): workgroup = (token, RH query heads of ONE key/value head, so one pass over
@@ -34,6 +38,7 @@ struct AttnPrep {
   float temp_coef;
   int temp_every;
   float eps;
+  UmbValueMix mix;                         // first: values to mix in; keep: where this layer's own go (fp32 rows of G E); null: neither
 };
 
 template <typename P>
@@ -61,8 +66,15 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(float* __restrict__ q, U
   }
   const int p = pos[t];
   if (is_v) {
-    El_* row = reinterpret_cast<El_*>(kv.v) + pkv_tok(kv, slot[t], p, hs - a.HQ - a.GK, a.G, a.E);
-    for (int i = lane; i < n; i += 64) stf<P>(row + i, src[i] * f);
+    const int g = hs - a.HQ - a.GK;
+    El_* row = reinterpret_cast<El_*>(kv.v) + pkv_tok(kv, slot[t], p, g, a.G, a.E);
+    const long o = ((long)t * a.G + g) * a.E;
+    for (int i = lane; i < n; i += 64) {
+      float v = src[i] * f;
+      if (a.mix.keep) a.mix.keep[o + i] = v;
+      if (a.mix.first) v = (1.f - a.mix.lambda) * v + a.mix.lambda * a.mix.first[o + i];
+      stf<P>(row + i, v);
+    }
     return;
   }
   const El_* w = is_q ? w_q : w_k;
@@ -125,7 +137,8 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
   __syncthreads();
   int j_lo = i - window + 1 > 0 ? i - window + 1 : 0;
   if (form.chunk > 0) j_lo = max(j_lo, i / form.chunk * form.chunk);
-  const int n_keys = i - j_lo + 1;
+  const int kept = min(form.keep_first, j_lo);          // first positions in front of the walk: keys 0 .. kept - 1, then j_lo .. i
+  const int n_keys = kept + i - j_lo + 1;
   const bool vec = (D & 7) == 0 && sizeof(El_) == 2;
   float acc[RH][NC], m_run[RH], l_run[RH];
 #pragma unroll
@@ -146,7 +159,7 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
     long off = 0;
     int dist = 0;
     if (kx < n_keys) {
-      const int j = j_lo + kx;
+      const int j = kx < kept ? kx : j_lo + kx - kept;
       dist = i - j;
       const El_* kr = reinterpret_cast<const El_*>(kv.k) + pkv_tok(kv, slot, j, g, G, MAPS * D);
       off = pkv_tok(kv, slot, j, g, G, E);
@@ -251,7 +264,9 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
     }
     return o;
   };
-  auto gate_of = [&](int h) { return gate_col >= 0 ? 1.f / (1.f + expf(-proj[(long)t * ld + gate_col + h])) : 1.f; };
+  auto gate_of = [&](int h, int d) {
+    return gate_col >= 0 ? 1.f / (1.f + expf(-proj[(long)t * ld + gate_col + (form.gate_elem ? h * E + d : h)])) : 1.f;
+  };
   if (MAPS == 1 || nsplit > 1) {
     for (int x = threadIdx.x; x < RH * E; x += NW * 64) {
       const int r = x / E, d = x % E;
@@ -264,7 +279,7 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
         continue;
       }
       if (form.sink) L += expf(form.sink[h0 + r] - M);
-      stf<P>(out + (long)t * ldo + (long)(h0 + r) * E + d, out_scale * gate_of(h0 + r) * (o / L));
+      stf<P>(out + (long)t * ldo + (long)(h0 + r) * E + d, out_scale * gate_of(h0 + r, d) * (o / L));
     }
   } else {
     // a wave per head: o = a1 - lambda a2 over its root mean square
@@ -283,10 +298,10 @@ __global__ __launch_bounds__(NW * 64) void bsa_attend_kernel(typename El<P>::typ
         if (lane + 64 * c < E) ss += o * o;
       }
       ss = wave_sum(ss);
-      const float f = out_scale * gate_of(h0 + rr) / sqrtf(ss / (float)E + form.eps);
+      const float f = out_scale / sqrtf(ss / (float)E + form.eps);
 #pragma unroll
       for (int c = 0; c < NC; ++c)
-        if (lane + 64 * c < E) stf<P>(out + (long)t * ldo + (long)(h0 + rr) * E + lane + 64 * c, v[c] * f);
+        if (lane + 64 * c < E) stf<P>(out + (long)t * ldo + (long)(h0 + rr) * E + dcl[c], v[c] * f * gate_of(h0 + rr, dcl[c]));
     }
   }
 }
@@ -298,7 +313,9 @@ __global__ __launch_bounds__(64) void bsa_merge_kernel(typename El<P>::type* __r
                                                        const float* __restrict__ proj, int ld, int gate_col, int H, int E,
                                                        int nsplit, float out_scale, UmbAttnForm form) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
-  const float gt = gate_col >= 0 ? 1.f / (1.f + expf(-proj[(long)t * ld + gate_col + h])) : 1.f;
+  auto gate_of = [&](int d) {
+    return gate_col >= 0 ? 1.f / (1.f + expf(-proj[(long)t * ld + gate_col + (form.gate_elem ? h * E + d : h)])) : 1.f;
+  };
   const float* pr[MAPS];
   float f[MAPS][16], inv[MAPS];
 #pragma unroll
@@ -328,8 +345,7 @@ __global__ __launch_bounds__(64) void bsa_merge_kernel(typename El<P>::type* __r
   };
   typename El<P>::type* orow = out + (long)t * ldo + (long)h * E;
   if constexpr (MAPS == 1) {
-    const float c = out_scale * gt;
-    for (int d = lane; d < E; d += 64) stf<P>(orow + d, column(0, d) * c);
+    for (int d = lane; d < E; d += 64) stf<P>(orow + d, column(0, d) * (out_scale * gate_of(d)));
   } else {
     float v[BSA_MAXC], ss = 0.f;
 #pragma unroll
@@ -342,25 +358,26 @@ __global__ __launch_bounds__(64) void bsa_merge_kernel(typename El<P>::type* __r
       }
     }
     ss = wave_sum(ss);
-    const float c0 = out_scale * gt / sqrtf(ss / (float)E + form.eps);
+    const float c0 = out_scale / sqrtf(ss / (float)E + form.eps);
 #pragma unroll
     for (int c = 0; c < BSA_MAXC; ++c)
-      if (lane + 64 * c < E) stf<P>(orow + lane + 64 * c, v[c] * c0);
+      if (lane + 64 * c < E) stf<P>(orow + lane + 64 * c, v[c] * (c0 * gate_of(lane + 64 * c)));
   }
 }
 
-static inline bool form_ok(const UmbAttnForm* f) { return !f || ((f->maps == 1 || f->maps == 2) && f->chunk >= 0); }
+static inline bool form_ok(const UmbAttnForm* f) { return !f || ((f->maps == 1 || f->maps == 2) && f->chunk >= 0 && f->keep_first >= 0); }
+static inline int form_gate_cols(const UmbAttnForm& f, int H, int E) { return f.gate_elem ? H * E : H; }
 
-extern "C" int umb_attn_prep(float* q, const UmbPagedKV* kv, const float* proj, int ld, int append, const void* w_q, const void* w_k,
-                             int norm_qk, int norm_v, const int* pos, const int* slot, const float* freq, int rot_dims, int layout,
-                             float rot_mult, int T, int H, int G, int D, int E, int maps, float temp_coef, int temp_every, float eps,
-                             int dtype, hipStream_t st) {
+extern "C" int umb_attn_prep_mix(float* q, const UmbPagedKV* kv, const float* proj, int ld, int append, const void* w_q, const void* w_k,
+                                 int norm_qk, int norm_v, const int* pos, const int* slot, const float* freq, int rot_dims, int layout,
+                                 float rot_mult, int T, int H, int G, int D, int E, int maps, float temp_coef, int temp_every, float eps,
+                                 const UmbValueMix* mix, int dtype, hipStream_t st) {
   if (T < 1 || H < 1 || G < 1 || H % G || D < 1 || E < 1 || maps < 1 || maps > 2 || rot_dims < 0 || rot_dims > D || (rot_dims & 1) ||
       (rot_dims && !freq) || layout < 0 || layout > 1 || !q || (append && !bsa_kv_ok(kv)) || !proj || !pos || !slot ||
       ld < maps * H * D + (append ? maps * G * D + G * E : 0))
     return UMB_EINVAL;
   AttnPrep a{maps * H, append ? maps * G : 0, G, append ? G : 0, D, E, maps, norm_qk, norm_v, rot_dims, layout, rot_mult,
-             temp_coef, temp_every, eps};
+             temp_coef, temp_every, eps, mix ? *mix : UmbValueMix{nullptr, nullptr, 0.f, 0.f}};
   const UmbPagedKV none{};
   const long items = (long)T * (a.HQ + a.GK + a.GV);
   DISPATCH_SEQ_DTYPE(dtype, {
@@ -370,6 +387,14 @@ extern "C" int umb_attn_prep(float* q, const UmbPagedKV* kv, const float* proj, 
   })
   UMB_LAUNCH_CHECK();
   return UMB_OK;
+}
+
+extern "C" int umb_attn_prep(float* q, const UmbPagedKV* kv, const float* proj, int ld, int append, const void* w_q, const void* w_k,
+                             int norm_qk, int norm_v, const int* pos, const int* slot, const float* freq, int rot_dims, int layout,
+                             float rot_mult, int T, int H, int G, int D, int E, int maps, float temp_coef, int temp_every, float eps,
+                             int dtype, hipStream_t st) {
+  return umb_attn_prep_mix(q, kv, proj, ld, append, w_q, w_k, norm_qk, norm_v, pos, slot, freq, rot_dims, layout, rot_mult, T, H, G, D, E,
+                           maps, temp_coef, temp_every, eps, nullptr, dtype, st);
 }
 
 extern "C" int umb_bsa_prep(float* q, const UmbPagedKV* kv, const float* proj, int ld, const void* w_q, const void* w_k,
@@ -396,9 +421,10 @@ extern "C" int umb_attn_attend(void* out, int ldo, const float* q, const UmbPage
                                int window, float scale, float out_scale, float softcap, const UmbAttnForm* form_, float* scratch,
                                long scratch_floats, int dtype, hipStream_t st) {
   if (T < 1 || H < 1 || G < 1 || H % G || D < 1 || E < 1 || E > 64 * BSA_MAXC || window < 1 || !out || !q || !bsa_kv_ok(kv) ||
-      !pos || !slot || ldo < H * E || (bias && n_dist < 1) || (gate_col >= 0 && (!proj || ld < gate_col + H)) || !form_ok(form_))
+      !pos || !slot || ldo < H * E || (bias && n_dist < 1) || !form_ok(form_))
     return UMB_EINVAL;
-  const UmbAttnForm form = form_ ? *form_ : UmbAttnForm{1, 0, nullptr, 0.f, 0.f};
+  const UmbAttnForm form = form_ ? *form_ : UmbAttnForm{1, 0, nullptr, 0.f, 0.f, 0, 0};
+  if (gate_col >= 0 && (!proj || ld < gate_col + form_gate_cols(form, H, E))) return UMB_EINVAL;
   const int maps = form.maps;
   const int hpg = H / G, nc = (E + 63) / 64;
   const int Dp = (D + 3) & ~3, Ep = (E + 3) & ~3, Mp = Dp > Ep ? Dp : Ep;
@@ -413,8 +439,9 @@ extern "C" int umb_attn_attend(void* out, int ldo, const float* q, const UmbPage
   int nsplit = 1;
   if (scratch && items <= 64) {                          // fewer than ~2048 waves in all with sixteen waves per item
     nsplit = (int)(512 / items) < 16 ? (int)(512 / items) : 16;
-    // keys of one chunk only: no more workgroups than there can be groups of four rounds
-    if (form.chunk > 0 && nsplit > (form.chunk + 255) / 256) nsplit = (form.chunk + 255) / 256;
+    // keys of one chunk or window only: no more workgroups than there can be groups of four rounds
+    const long most = (long)(form.chunk > 0 && form.chunk < window ? form.chunk : window) + form.keep_first;
+    if (nsplit > (most + 255) / 256) nsplit = (int)((most + 255) / 256);
     while (nsplit > 1 && (long)T * H * maps * nsplit * (E + 2) > scratch_floats) nsplit >>= 1;
   }
   const dim3 grid(T, hblocks, nsplit);
@@ -527,7 +554,9 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
     j_lo = max(j_lo, i_first / form.chunk * form.chunk);
     c_lo = i_j / form.chunk * form.chunk;
   }
-  const int total = i_last - j_lo + 1;
+  const int kept = min(form.keep_first, j_lo);        // first positions in front of the walk: step rows 0 .. kept - 1, then j_lo .. i_last
+  const int j_off = j_lo - kept;
+  const int total = kept + i_last - j_lo + 1;
   const float scale2 = scale * BSA_LOG2E;
   const u16* kbase = reinterpret_cast<const u16*>(kv.k);
   const u16* vbase = reinterpret_cast<const u16*>(kv.v);
@@ -568,8 +597,9 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
   auto fetch = [&](int base) {
     const int kx = base + sm;
     const bool ok = kx < total;
-    const long offk = ok ? pkv_tok(kv, slot, j_lo + kx, g, G, DK) : 0;
-    const long offv = ok ? pkv_tok(kv, slot, j_lo + kx, g, G, E) : 0;
+    const int jk = kx < kept ? kx : j_off + kx;
+    const long offk = ok ? pkv_tok(kv, slot, jk, g, G, DK) : 0;
+    const long offv = ok ? pkv_tok(kv, slot, jk, g, G, E) : 0;
 #pragma unroll
     for (int u = 0; u < NLK; ++u) {
       const int ch = sc + 8 * u;
@@ -608,8 +638,9 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
     int di[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      const int jt = j_lo + base + 16 * (e >> 2) + 4 * g4 + (e & 3);
-      vis[e] = q_ok && jt <= i_j && jt > i_j - window && jt >= c_lo;
+      const int kx = base + 16 * (e >> 2) + 4 * g4 + (e & 3);
+      const int jt = kx < kept ? kx : j_off + kx;
+      vis[e] = q_ok && jt <= i_j && ((jt > i_j - window && jt >= c_lo) || jt < form.keep_first);
       const int dd = i_j - jt;
       di[e] = dd < 0 ? 0 : (dd < n_dist ? dd : n_dist - 1);
     }
@@ -699,7 +730,9 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
 #pragma unroll
     for (int hh = 0; hh < HPW; hh += MAPS) {
       if (!h_ok[hh]) continue;
-      const float gt = gate_col >= 0 ? 1.f / (1.f + expf(-proj[qrow * ld + gate_col + hd[hh]])) : 1.f;
+      const bool gate_head = gate_col >= 0 && !form.gate_elem;
+      const float gt = gate_head ? 1.f / (1.f + expf(-proj[qrow * ld + gate_col + hd[hh]])) : 1.f;
+      const float* ge = gate_col >= 0 && form.gate_elem ? proj + qrow * ld + gate_col + (long)hd[hh] * E : nullptr;
       float l[MAPS];
 #pragma unroll
       for (int mp = 0; mp < MAPS; ++mp)
@@ -728,7 +761,12 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
       for (int dt = 0; dt < NVM; ++dt) {
         if (dt < nv) {
 #pragma unroll
-          for (int rr = 0; rr < 4; ++rr) orow[16 * dt + 4 * g4 + rr] = P::from_f(o[hh][dt][rr] * inv);
+          for (int rr = 0; rr < 4; ++rr) {
+            const int d = 16 * dt + 4 * g4 + rr;
+            float v = o[hh][dt][rr] * inv;
+            if (ge) v /= 1.f + expf(-ge[d]);
+            orow[d] = P::from_f(v);
+          }
         }
       }
     }
@@ -746,11 +784,11 @@ extern "C" int umb_attn_attend_tiled(void* out, int ldo, const float* q, const U
                                      int window, float scale, float out_scale, float softcap, const UmbAttnForm* form_, int dtype,
                                      hipStream_t st) {
   if (B < 1 || B > 65535 || max_len < 1 || window < 1 || !out || !q || !bsa_kv_ok(kv) || !seq_slot || !seq_row0 || !seq_pos0 ||
-      !seq_len || ldo < H * E || (bias && n_dist < 1) || (gate_col >= 0 && (!proj || ld < gate_col + H)) ||
-      !umb_bsa_attend_tiled_ok(H, G, D, E, dtype) || !form_ok(form_))
+      !seq_len || ldo < H * E || (bias && n_dist < 1) || !umb_bsa_attend_tiled_ok(H, G, D, E, dtype) || !form_ok(form_))
     return UMB_EINVAL;
   if (!bias) n_dist = 1;
-  const UmbAttnForm form = form_ ? *form_ : UmbAttnForm{1, 0, nullptr, 0.f, 0.f};
+  const UmbAttnForm form = form_ ? *form_ : UmbAttnForm{1, 0, nullptr, 0.f, 0.f, 0, 0};
+  if (gate_col >= 0 && (!proj || ld < gate_col + form_gate_cols(form, H, E))) return UMB_EINVAL;
   const int hpg = H / G, maps = form.maps;
   const size_t lds = ((size_t)32 * (maps * D + 8) + (size_t)E * 36) * sizeof(u16);
 #define BSA_MFMA(NSM, NVM, HPW, MAPS)                                                                                      \

@@ -11,8 +11,11 @@
 //
 // Visibility: position i sees j with 0 <= i - j < window.  Softmax with a sink: the denominator also holds exp(sink[h]),
 // which has no key and no value and is not scaled.  Scores, weights, maxima and sums are fp32; rotary angles are
-// pos * freq[i] in fp32 through the full-range sincosf; pairs (2i, 2i+1) of the first rot_dims features of the rotated part
-// turn, the rest pass.
+// pos * freq[i] in fp32 through the full-range sincosf; of the rotated part's first rot_dims features the pairs (2i, 2i+1), or
+// (i, i + rot_dims / 2) in the other layout, turn (cos and sin times a constant), the rest pass.
+//
+// Two front ends: queries through a latent of their own (lat_prep norms both latents and appends, an up-projection follows,
+// lat_qsplit takes its result apart), or queries straight from the fused input projection (lat_front: one launch for all of it).
 #include "seq_common.h"
 #include <cstdlib>
 
@@ -85,6 +88,81 @@ __global__ __launch_bounds__(256) void lat_qsplit_kernel(typename El<P>::type* _
     const float ru = u * cs - v * sn, rv = v * cs + u * sn;
     u = ru; v = rv;
   }
+  float* dst = qa + th * (kv_rank + R) + kv_rank;
+  dst[d0] = u;
+  if (d1 < R) dst[d1] = v;
+}
+
+// ---- queries straight from the input projection, one launch: workgroup (token, 0) norms the latent, turns the shared key part and
+// appends the row; workgroups (token, 1 ..) take 256 items of the token's queries each -- four unrotated features (converted for the
+// product with W_uk^T) or one feature pair of the rotated part.
+template <typename P>
+__global__ __launch_bounds__(256) void lat_front_kernel(typename El<P>::type* __restrict__ qn, float* __restrict__ qa, UmbPagedKV kv,
+                                                        const float* __restrict__ proj, int ld, int q_col, int kv_col,
+                                                        const typename El<P>::type* __restrict__ w_kv, const int* __restrict__ pos,
+                                                        const int* __restrict__ slot, const float* __restrict__ freq, int H, int D, int R,
+                                                        int kv_rank, int rot_dims, int layout, float rot_mult, float eps) {
+  typedef typename El<P>::type E;
+  __shared__ float red[8];
+  const int t = blockIdx.x, p = pos[t], half = rot_dims >> 1;
+  const float pf = (float)p;
+  // pair m of a rotated part: features d0, d1 (d1 >= R: a single feature left over), turned if m < half
+  auto pair_of = [&](int m, int& d0, int& d1) {
+    if (m < half) { d0 = layout == 0 ? m : 2 * m; d1 = layout == 0 ? m + half : 2 * m + 1; }
+    else { d0 = rot_dims + 2 * (m - half); d1 = d0 + 1; }
+  };
+  auto turn = [&](int m, float& u, float& v) {
+    if (m >= half) return;
+    float sn, cs;
+    sincosf(pf * freq[m], &sn, &cs);
+    sn *= rot_mult;
+    cs *= rot_mult;
+    const float ru = u * cs - v * sn, rv = v * cs + u * sn;
+    u = ru;
+    v = rv;
+  };
+  const int pairs = (R + 1) / 2;
+  if (blockIdx.y == 0) {
+    const float* src = proj + (long)t * ld + kv_col;
+    float ss = 0.f;
+#pragma unroll 4
+    for (int i = threadIdx.x; i < kv_rank; i += 256) { const float v = src[i]; ss += v * v; }
+    ss = block_sum<256>(ss, red);
+    const float f = 1.f / sqrtf(ss / (float)kv_rank + eps);
+    E* row = reinterpret_cast<E*>(kv.k) + pkv_tok(kv, slot[t], p, 0, 1, kv_rank + R);
+    for (int i = threadIdx.x; i < kv_rank; i += 256) stf<P>(row + i, src[i] * f * ldf<P>(w_kv + i));
+    const float* kr = src + kv_rank;
+    for (int m = threadIdx.x; m < pairs; m += 256) {
+      int d0, d1;
+      pair_of(m, d0, d1);
+      float u = kr[d0], v = d1 < R ? kr[d1] : 0.f;
+      turn(m, u, v);
+      stf<P>(row + kv_rank + d0, u);
+      if (d1 < R) stf<P>(row + kv_rank + d1, v);
+    }
+    return;
+  }
+  const int quads = (D + 3) / 4, per = quads + pairs;
+  const int item = (blockIdx.y - 1) * 256 + threadIdx.x;
+  if (item >= H * per) return;
+  const int h = item / per, e = item % per;
+  const float* src = proj + (long)t * ld + q_col + (long)h * (D + R);
+  const long th = (long)t * H + h;
+  if (e < quads) {
+    const int d = 4 * e, n = D - d < 4 ? D - d : 4;
+    float v[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = i < n ? src[d + i] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (i < n) stf<P>(qn + th * D + d + i, v[i]);
+    return;
+  }
+  const int m = e - quads;
+  int d0, d1;
+  pair_of(m, d0, d1);
+  float u = src[D + d0], v = d1 < R ? src[D + d1] : 0.f;
+  turn(m, u, v);
   float* dst = qa + th * (kv_rank + R) + kv_rank;
   dst[d0] = u;
   if (d1 < R) dst[d1] = v;
@@ -651,6 +729,24 @@ extern "C" int umb_lat_qsplit(void* qn, float* qa, const float* q, const int* po
     typedef typename El<P>::type E;
     hipLaunchKernelGGL(lat_qsplit_kernel<P>, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, (E*)qn, qa, q, pos, freq, T, H,
                        D, R, kv_rank, rot_dims);
+  })
+  UMB_LAUNCH_CHECK();
+  return UMB_OK;
+}
+
+extern "C" int umb_lat_front(void* qn, float* qa, const UmbPagedKV* kv, const float* proj, int ld, int q_col, int kv_col, const void* w_kv,
+                             const int* pos, const int* slot, const float* freq, int T, int H, int D, int R, int kv_rank, int rot_dims,
+                             int layout, float rot_mult, float eps, int dtype, hipStream_t st) {
+  if (T < 1 || H < 1 || D < 1 || R < 0 || kv_rank < 1 || rot_dims < 0 || rot_dims > R || (rot_dims & 1) || layout < 0 || layout > 1 ||
+      !qn || !qa || !lat_kv_ok(kv) || !proj || !w_kv || !pos || !slot || (rot_dims && !freq) || q_col < 0 || kv_col < 0 ||
+      ld < q_col + H * (D + R) || ld < kv_col + kv_rank + R)
+    return UMB_EINVAL;
+  const long items = (long)H * ((D + 3) / 4 + (R + 1) / 2);
+  if ((items + 255) / 256 + 1 > 65535) return UMB_EINVAL;
+  DISPATCH_SEQ_DTYPE(dtype, {
+    typedef typename El<P>::type E;
+    hipLaunchKernelGGL(lat_front_kernel<P>, dim3(T, (unsigned)((items + 255) / 256 + 1)), dim3(256), 0, st, (E*)qn, qa, *kv, proj, ld, q_col,
+                       kv_col, (const E*)w_kv, pos, slot, freq, H, D, R, kv_rank, rot_dims, layout, rot_mult, eps);
   })
   UMB_LAUNCH_CHECK();
   return UMB_OK;

@@ -56,29 +56,37 @@ template <> __device__ __forceinline__ f32x4 mma8<F32>(const Frag8<F32>& a, cons
   return c;
 }
 
-enum { EPI_F32 = 0, EPI_DT = 1, EPI_SILU_MUL = 2, EPI_GATE = 3, EPI_RELU2 = 4, EPI_CLAMP_GLU = 5 };
-// the two stacked-halves epilogues: silu(gate) * up, or the capped form g sigmoid(alpha g) (u + 1) with g = min(gate, limit),
-// u = clamp(up, -limit, limit)
-static inline bool epi_dual(int epi) { return epi == EPI_SILU_MUL || epi == EPI_CLAMP_GLU; }
+enum { EPI_F32 = 0, EPI_DT = 1, EPI_SILU_MUL = 2, EPI_GATE = 3, EPI_RELU2 = 4, EPI_CLAMP_GLU = 5, EPI_GELU_MUL = 6, EPI_GATE_ROW = 7, EPI_CAP = 8 };
+// the stacked-halves epilogues: silu(gate) * up, gelu(gate) * up (tanh form), or the capped form g sigmoid(alpha g) (u + 1) with
+// g = min(gate, limit), u = clamp(up, -limit, limit)
+static inline bool epi_dual(int epi) { return epi == EPI_SILU_MUL || epi == EPI_CLAMP_GLU || epi == EPI_GELU_MUL; }
+// epilogues that umb_seq_linear / umb_seq_linear_grouped take by number (the others have constants or a gate of their own)
+static inline bool epi_plain(int epi) {
+  return epi == EPI_F32 || epi == EPI_DT || epi == EPI_SILU_MUL || epi == EPI_RELU2 || epi == EPI_GELU_MUL;
+}
+// 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))
+__device__ __forceinline__ float gelu_tanhf_(float z) { return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 __device__ __forceinline__ float glu_pair(int epi, float g, float u, float limit, float alpha) {
   if (epi == EPI_CLAMP_GLU) {
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
     return g / (1.f + expf(-alpha * g)) * (u + 1.f);
   }
+  if (epi == EPI_GELU_MUL) return gelu_tanhf_(g) * u;
   return siluf_(g) * u;
 }
 
 // Where a launch departs from the dense [T][K] x [N][K] problem: row strides of x and out, a batch of independent problems
 // along blockIdx.z (element strides sx / sw / so), or token tiles read from device memory (grouped: tile blockIdx.y is
-// {group, first row, rows}; its weights start at w + group * gs).  EPI_GATE multiplies by sigmoid(gate[t ldg + z sg + n]).
+// {group, first row, rows}; its weights start at w + group * gs).  EPI_GATE multiplies by sigmoid(gate[t ldg + z sg + n]),
+// EPI_GATE_ROW by sigmoid(gate[t ldg + z sg]): one number per row and problem.
 struct LinExt {
   int ldx, ldo;
   long sx, sw, so, gs;
   const int* tiles;
   const float* gate;
   int ldg, sg;
-  float limit, alpha;      // EPI_CLAMP_GLU
+  float limit, alpha;      // EPI_CLAMP_GLU; EPI_CAP: out = limit tanh(acc / limit), fp32
 };
 static inline LinExt lin_dense(int N, int K) { return LinExt{K, N, 0, 0, 0, 0, nullptr, nullptr, 0, 0}; }
 
@@ -201,6 +209,10 @@ __global__ __launch_bounds__(256) void seq_linear_kernel(void* __restrict__ out_
         stf<P>(reinterpret_cast<E*>(out_) + obase + (long)t * ldo + n, rl * rl);
       } else if (epi == EPI_GATE) {
         stf<P>(reinterpret_cast<E*>(out_) + obase + (long)t * ldo + n, s / (1.f + expf(-gate[(long)t * ext.ldg + n])));
+      } else if (epi == EPI_GATE_ROW) {
+        stf<P>(reinterpret_cast<E*>(out_) + obase + (long)t * ldo + n, s / (1.f + expf(-gate[(long)t * ext.ldg])));
+      } else if (epi == EPI_CAP) {
+        reinterpret_cast<float*>(out_)[obase + (long)t * ldo + n] = ext.limit * tanhf(s / ext.limit);
       } else {
         reinterpret_cast<float*>(out_)[obase + (long)t * ldo + n] = s;
       }
@@ -319,6 +331,8 @@ __global__ __launch_bounds__(256) void seq_linear_wide_kernel(void* __restrict__
         } else if (epi == EPI_RELU2) {
           const float rl = fmaxf(sv, 0.f);
           reinterpret_cast<u16*>(out_)[obase + (long)t * N + n] = P::from_f(rl * rl);
+        } else if (epi == EPI_CAP) {
+          reinterpret_cast<float*>(out_)[obase + (long)t * N + n] = ext.limit * tanhf(sv / ext.limit);
         } else {
           reinterpret_cast<float*>(out_)[obase + (long)t * N + n] = sv;
         }
@@ -369,7 +383,7 @@ static int launch_vec(void* out, const void* x, const void* w, const void* bias,
   if (T <= 32) return launch_tt<P, 1, 2, VEC>(out, x, w, bias, T, N, K, epi, st, ext, 0, gz);
   // many tokens: the launch is bound by fragment loads per MFMA, not by weight bytes -> four output tiles per workgroup
   // (the K order of every output is unchanged: a row's value does not depend on which variant computed it)
-  const bool dense = gz == 1 && ext.ldx == K && ext.ldo == N && epi != EPI_GATE;
+  const bool dense = gz == 1 && ext.ldx == K && ext.ldo == N && epi != EPI_GATE && epi != EPI_GATE_ROW;
   if (T > 64 && N >= 64 && sizeof(typename El<P>::type) == 2) {
     if (VEC && dense && T >= 256 && N >= 128) return launch_wide<P>(out, x, w, bias, T, N, K, epi, st, LinExt{0, 0, 0, 0, 0, 0, nullptr, nullptr, 0, 0, ext.limit, ext.alpha});      // both operands re-used
     return launch_tt<P, 4, 4, VEC>(out, x, w, bias, T, N, K, epi, st, ext, 0, gz);
@@ -379,7 +393,7 @@ static int launch_vec(void* out, const void* x, const void* w, const void* bias,
 
 static int seq_linear_any(void* out, const void* x, const void* w, const void* bias, int T, int N, int K, int epi, float limit,
                           float alpha, int dtype, hipStream_t st) {
-  if (T < 1 || N < 1 || K < 1 || epi < 0 || (epi > 2 && epi != EPI_RELU2 && epi != EPI_CLAMP_GLU) || !out || !x || !w) return UMB_EINVAL;
+  if (T < 1 || N < 1 || K < 1 || !(epi_plain(epi) || epi == EPI_CLAMP_GLU || epi == EPI_CAP) || !out || !x || !w) return UMB_EINVAL;
   if (epi_dual(epi)) {
     if (N & 1) return UMB_EINVAL;
     N >>= 1;                                   // rows of each half
@@ -395,7 +409,7 @@ static int seq_linear_any(void* out, const void* x, const void* w, const void* b
 
 extern "C" int umb_seq_linear(void* out, const void* x, const void* w, const void* bias, int T, int N, int K, int epi, int dtype,
                               hipStream_t st) {
-  if (epi == EPI_CLAMP_GLU) return UMB_EINVAL;              // that epilogue has constants: umb_seq_linear_glu
+  if (!epi_plain(epi)) return UMB_EINVAL;                   // the others have constants: umb_seq_linear_glu, umb_seq_linear_cap
   return seq_linear_any(out, x, w, bias, T, N, K, epi, 0.f, 0.f, dtype, st);
 }
 
@@ -405,11 +419,17 @@ extern "C" int umb_seq_linear_glu(void* out, const void* x, const void* w, const
   return seq_linear_any(out, x, w, bias, T, N, K, EPI_CLAMP_GLU, limit, alpha, dtype, st);
 }
 
+extern "C" int umb_seq_linear_cap(void* out, const void* x, const void* w, const void* bias, int T, int N, int K, float cap, int dtype,
+                                  hipStream_t st) {
+  if (!(cap > 0.f)) return UMB_EINVAL;
+  return seq_linear_any(out, x, w, bias, T, N, K, EPI_CAP, cap, 0.f, dtype, st);
+}
+
 extern "C" int umb_seq_linear_batched(void* out, const void* x, const void* w, int T, int N, int K, int ldx, int ldo, int batch,
                                       long sx, long sw, long so, int epi, const float* gate, int ldg, int sg, int dtype,
                                       hipStream_t st) {
   if (T < 1 || N < 1 || K < 1 || batch < 1 || batch > 65535 || ldx < K || ldo < N || !out || !x || !w ||
-      !(epi == EPI_F32 || epi == EPI_DT || epi == EPI_GATE) || (epi == EPI_GATE && !gate))
+      !(epi == EPI_F32 || epi == EPI_DT || epi == EPI_GATE || epi == EPI_GATE_ROW) || ((epi == EPI_GATE || epi == EPI_GATE_ROW) && !gate))
     return UMB_EINVAL;
   const LinExt ext{ldx, ldo, sx, sw, so, 0, nullptr, gate, ldg, sg};
   // 16-byte loads need every row start aligned: the strides as well as K
@@ -422,7 +442,7 @@ extern "C" int umb_seq_linear_batched(void* out, const void* x, const void* w, i
 
 static int seq_linear_grouped_any(void* out, const void* x, const void* w, const int* tiles, int max_tiles, int tile_rows, long gs,
                                   int N, int K, int epi, float limit, float alpha, int dtype, hipStream_t st) {
-  if (max_tiles < 1 || max_tiles > 65535 || N < 1 || K < 1 || epi < 0 || (epi > 2 && epi != EPI_RELU2 && epi != EPI_CLAMP_GLU) || !out ||
+  if (max_tiles < 1 || max_tiles > 65535 || N < 1 || K < 1 || !(epi_plain(epi) || epi == EPI_CLAMP_GLU) || !out ||
       !x || !w || !tiles ||
       (tile_rows != 16 && tile_rows != 64 && tile_rows != 128))
     return UMB_EINVAL;
@@ -453,7 +473,7 @@ static int seq_linear_grouped_any(void* out, const void* x, const void* w, const
 
 extern "C" int umb_seq_linear_grouped(void* out, const void* x, const void* w, const int* tiles, int max_tiles, int tile_rows,
                                       long gs, int N, int K, int epi, int dtype, hipStream_t st) {
-  if (epi == EPI_CLAMP_GLU) return UMB_EINVAL;
+  if (!epi_plain(epi)) return UMB_EINVAL;
   return seq_linear_grouped_any(out, x, w, tiles, max_tiles, tile_rows, gs, N, K, epi, 0.f, 0.f, dtype, st);
 }
 

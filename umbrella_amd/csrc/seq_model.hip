@@ -16,6 +16,7 @@
 //     differential attention: proj GEMM ([q | k | v], or [q] over another layer's store) | rotary + append | attend + combine | out GEMM
 //     attention with a sink beside a gated delta rule (one fused proj GEMM): norms + append | attend  ||  convolution + unit norms +
 //                gates | ring | chunk solve | chunk scan (single tokens: one launch) | per-head norm * SiLU gate | two out GEMMs | pair seam
+//     softmax attention by form: proj GEMM ([q | k | v | gate]) | norms or rotary + value mixing + append | attend (bias, sink, gate) | out GEMM
 // Stacks whose two sublayers read the SAME residual (UmbSeqModel.block = UMB_BLOCK_PARALLEL) run mixer and feed-forward from two
 // normed inputs and meet in one seam per layer; a layer may ask for the embedding row to be added again in front of it.
 // Models with several residual streams (UmbSeqModel.streams >= 1) use the stream seam instead: write of the sublayer behind
@@ -63,18 +64,19 @@ static int seam(const UmbSeqModel* m, const UmbSeqWork* ws, const UmbSeqStep* s,
   return umb_seq_resid_norm(ws->x, ws->h, ws->y, w_post, w_next, T, W, m->groups, m->eps, m->dtype, st);
 }
 
-// the first product of a feed-forward with its activation as epilogue: silu(gate) * up or the capped form over stacked
-// [gate; up], or relu(up)^2
+// the first product of a feed-forward with its activation as epilogue: silu(gate) * up, gelu(gate) * up or the capped form over
+// stacked [gate; up], or relu(up)^2
+static int act_epi(int act) { return act == UMB_ACT_RELU2 ? 4 : (act == UMB_ACT_GELU_GATED ? 6 : 2); }
 static int lin_act(const UmbSeqLayer& ly, const UmbSeqLinear& l, float limit, void* out, const void* x, int T, int dt, hipStream_t st) {
   if (ly.act_kind == UMB_ACT_CLAMP_GLU) return umb_seq_linear_glu(out, x, l.w, l.bias, T, l.N, l.K, limit, ly.act_alpha, dt, st);
-  return lin(l, out, x, T, ly.act_kind == UMB_ACT_RELU2 ? 4 : 2, dt, st);
+  return lin(l, out, x, T, act_epi(ly.act_kind), dt, st);
 }
 
 // feed-forward of h_in (dtype [T][W]) into y_out (fp32 [T][W])
 static int feed_forward(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWork* ws, const UmbSeqStep* s, const void* h_in,
                         float* y_out, hipStream_t st) {
   const int T = s->T, W = m->W, dt = m->dtype;
-  const int epi = ly.act_kind == UMB_ACT_RELU2 ? 4 : 2, stack = ly.act_kind == UMB_ACT_RELU2 ? 1 : 2;
+  const int epi = act_epi(ly.act_kind), stack = ly.act_kind == UMB_ACT_RELU2 ? 1 : 2;
   if (ly.ff_kind == UMB_FF_GATED) {
     SEQ_TRY(lin_act(ly, ly.gu, ly.act_limit, ws->act, h_in, T, dt, st));
     return lin(ly.down, y_out, ws->act, T, 0, dt, st);
@@ -266,13 +268,33 @@ static int mix_attn_mlstm(const UmbSeqModel* m, const UmbSeqLayer& ly, const Umb
 }
 
 // the two places attention mixers meet the keys: the matrix pipe for steps that bring stretches, the vector pipe otherwise
+// (gate_col: first column of the output gate in proj, -1: none)
 static int attend(const UmbSeqLayer& ly, void* out, const float* q, const UmbSeqStep* s, int H, int G, int D, int E, int window,
-                  float out_scale, const UmbAttnForm& form, float* scratch, long scratch_floats, int dt, hipStream_t st) {
+                  float out_scale, const UmbAttnForm& form, float* scratch, long scratch_floats, int dt, hipStream_t st,
+                  const float* proj = nullptr, int ld = 0, int gate_col = -1) {
   if (s->max_len >= 16 && umb_bsa_attend_tiled_ok(H, G, D, E, dt))
-    return umb_attn_attend_tiled(out, H * E, q, &ly.kv, nullptr, 0, -1, nullptr, 0, s->seq_slot, s->seq_row0, s->seq_pos0, s->seq_len, s->B,
-                                 s->max_len, H, G, D, E, window, ly.scale, out_scale, 0.f, &form, dt, st);
-  return umb_attn_attend(out, H * E, q, &ly.kv, nullptr, 0, -1, nullptr, 0, s->pos, s->slot, s->T, H, G, D, E, window, ly.scale, out_scale,
-                         0.f, &form, scratch_floats > 0 ? scratch : nullptr, scratch_floats, dt, st);
+    return umb_attn_attend_tiled(out, H * E, q, &ly.kv, proj, ld, gate_col, ly.dist_bias, ly.n_dist, s->seq_slot, s->seq_row0, s->seq_pos0,
+                                 s->seq_len, s->B, s->max_len, H, G, D, E, window, ly.scale, out_scale, 0.f, &form, dt, st);
+  return umb_attn_attend(out, H * E, q, &ly.kv, proj, ld, gate_col, ly.dist_bias, ly.n_dist, s->pos, s->slot, s->T, H, G, D, E, window, ly.scale,
+                         out_scale, 0.f, &form, scratch_floats > 0 ? scratch : nullptr, scratch_floats, dt, st);
+}
+
+// softmax attention by form: one map; norms, rotary, bias by distance, window with kept first tokens or chunks, sink, element-wise
+// gate and value mixing, each where the layer asks for it
+static int mix_softmax(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWork* ws, const UmbSeqStep* s, hipStream_t st) {
+  const int T = s->T, dt = m->dtype, ld = ly.proj.N, H = ly.heads, G = ly.kv_heads, D = ly.dim, E = ly.vdim;
+  const int gate_col = H * D + G * (D + E);
+  if (H < 1 || G < 1 || ld != gate_col + (ly.gate_elem ? H * E : 0) || ly.out.K != H * E || !ly.q_norm != !ly.k_norm ||
+      ly.v_mix < 0 || ly.v_mix > 2 || (ly.v_mix && !ws->v_first))
+    return UMB_EINVAL;
+  float* q = ws->aux;                                        // [T][H D] | scratch
+  float* spare = q + al4((long)T * H * D);
+  const UmbValueMix mix{ly.v_mix == 2 ? ws->v_first : nullptr, ly.v_mix == 1 ? ws->v_first : nullptr, ly.v_lambda, 0.f};
+  SEQ_TRY(umb_attn_prep_mix(q, &ly.kv, ws->proj, ld, 1, ly.q_norm, ly.k_norm, ly.q_norm != nullptr, 0, s->pos, s->slot, ly.rot_freq, ly.rot_dims,
+                            ly.rot_layout, ly.rot_mult, T, H, G, D, E, 1, 0.f, 0, m->eps, &mix, dt, st));
+  const UmbAttnForm form{1, ly.chunk, ly.attn_sink, 0.f, 0.f, ly.keep_first, ly.gate_elem};
+  return attend(ly, ws->mix, q, s, H, G, D, E, ly.window, 1.f, form, spare, ws->aux_floats - (long)(spare - ws->aux), dt, st, ws->proj, ld,
+                ly.gate_elem ? gate_col : -1);
 }
 
 // differential attention: two maps per head over the same values; with kv_shared the keys and values are another layer's
@@ -283,7 +305,7 @@ static int mix_diff_attn(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbS
   float* spare = q + al4((long)T * 2 * H * D);
   SEQ_TRY(umb_attn_prep(q, &ly.kv, ws->proj, ld, !ly.kv_shared, nullptr, nullptr, 0, 0, s->pos, s->slot, ly.rot_freq, ly.rot_dims,
                         ly.rot_layout, ly.rot_mult, T, H, G, D, E, 2, 0.f, 0, m->eps, dt, st));
-  const UmbAttnForm form{2, ly.chunk, nullptr, ly.diff_lambda, m->eps};
+  const UmbAttnForm form{2, ly.chunk, nullptr, ly.diff_lambda, m->eps, 0, 0};
   return attend(ly, ws->mix, q, s, H, G, D, E, ly.window, ly.out_mult, form, spare, ws->aux_floats - (long)(spare - ws->aux), dt, st);
 }
 
@@ -303,7 +325,7 @@ static int mix_attn_delta(const UmbSeqModel* m, const UmbSeqLayer& ly, const Umb
   float* spare = q + al4((long)T * H * D);
   SEQ_TRY(umb_attn_prep(q, &ly.kv, ws->proj, ld, 1, ly.q_norm, ly.k_norm, 1, 0, s->pos, s->slot, nullptr, 0, 0, 1.f, T, H, G, D, E, 1, 0.f, 0,
                         m->eps, dt, st));
-  const UmbAttnForm form{1, 0, ly.attn_sink, 0.f, 0.f};
+  const UmbAttnForm form{1, 0, ly.attn_sink, 0.f, 0.f, 0, 0};
   SEQ_TRY(attend(ly, ws->mix, q, s, H, G, D, E, ly.window, 1.f, form, spare, ws->aux_floats - (long)(spare - ws->aux), dt, st));
   if (s->max_len == 1)
     SEQ_TRY(umb_delta_step(ws->o, ly.state, ws->proj, ld, col0, ly.s_conv, ly.s_conv_state, ly.s_dt_bias, ly.s_a_log, s->pos, s->slot, T, Hk,
@@ -356,13 +378,20 @@ static int run_mixer(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWo
     // proj = [dq | dkv (latent + rotated key part) | gate]; the query latent goes up to the heads, its unrotated parts are
     // carried into the key/value latent space (W_uk^T, one product per head), attention runs against the cached rows, the
     // value up-projection W_uv follows the weighted sum, with the sigmoid gate as its epilogue
+    // (q_rank 0: the queries themselves stand in the projection, [q | dkv | gate])
     const int H = ly.heads, D = ly.dim, R = ly.rot_dim, Dv = ly.vdim, Rq = ly.q_rank, Rc = ly.kv_rank, Dk = Rc + R;
-    if (ld != Rq + Dk + H * Dv || ly.uq.N != H * (D + R) || ly.uq.K != Rq || !ly.uk_t || !ly.uv || !ly.dq_norm || !ly.dkv_norm)
-      return UMB_EINVAL;
-    SEQ_TRY(umb_lat_prep(ws->act, &ly.kv, ws->proj, ld, ly.dq_norm, ly.dkv_norm, s->pos, s->slot, ly.rot_freq, T, Rq, Rc, R,
-                         ly.rot_dims, eps, dt, st));
-    SEQ_TRY(lin(ly.uq, ws->o, ws->act, T, 0, dt, st));
-    SEQ_TRY(umb_lat_qsplit(ws->mix, ws->aux, ws->o, s->pos, ly.rot_freq, T, H, D, R, Rc, ly.rot_dims, dt, st));
+    const int kv_col = Rq > 0 ? Rq : H * (D + R), gate_col = kv_col + Dk, gates = ly.gate_head ? H : H * Dv;
+    if (ld != gate_col + gates || !ly.uk_t || !ly.uv || !ly.dkv_norm || ly.out.K != H * Dv) return UMB_EINVAL;
+    if (Rq > 0) {
+      if (ly.uq.N != H * (D + R) || ly.uq.K != Rq || !ly.dq_norm || ly.rot_layout != 1 || ly.rot_mult != 1.f) return UMB_EINVAL;
+      SEQ_TRY(umb_lat_prep(ws->act, &ly.kv, ws->proj, ld, ly.dq_norm, ly.dkv_norm, s->pos, s->slot, ly.rot_freq, T, Rq, Rc, R,
+                           ly.rot_dims, eps, dt, st));
+      SEQ_TRY(lin(ly.uq, ws->o, ws->act, T, 0, dt, st));
+      SEQ_TRY(umb_lat_qsplit(ws->mix, ws->aux, ws->o, s->pos, ly.rot_freq, T, H, D, R, Rc, ly.rot_dims, dt, st));
+    } else {
+      SEQ_TRY(umb_lat_front(ws->mix, ws->aux, &ly.kv, ws->proj, ld, 0, kv_col, ly.dkv_norm, s->pos, s->slot, ly.rot_freq, T, H, D, R, Rc,
+                            ly.rot_dims, ly.rot_layout, ly.rot_mult, eps, dt, st));
+    }
     SEQ_TRY(umb_seq_linear_batched(ws->aux, ws->mix, ly.uk_t, T, Rc, D, H * D, H * Dk, H, D, (long)Rc * D, Dk, 0, nullptr, 0, 0,
                                    dt, st));
     if (s->max_len >= 16 && umb_lat_attend_tiled_ok(H, Rc, R, dt))
@@ -370,8 +399,8 @@ static int run_mixer(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWo
                                    s->max_len, H, Rc, R, ly.window, ly.scale, dt, st));
     else
       SEQ_TRY(umb_lat_attend(ws->act, ws->aux, &ly.kv, ly.sink, s->pos, s->slot, T, H, Rc, R, ly.window, ly.scale, dt, st));
-    SEQ_TRY(umb_seq_linear_batched(ws->mix, ws->act, ly.uv, T, Dv, Rc, H * Rc, H * Dv, H, Rc, (long)Dv * Rc, Dv, 3,
-                                   ws->proj + Rq + Dk, ld, Dv, dt, st));
+    SEQ_TRY(umb_seq_linear_batched(ws->mix, ws->act, ly.uv, T, Dv, Rc, H * Rc, H * Dv, H, Rc, (long)Dv * Rc, Dv, ly.gate_head ? 7 : 3,
+                                   ws->proj + gate_col, ld, ly.gate_head ? 1 : Dv, dt, st));
   } else if (ly.kind == UMB_MIX_MINGRU) {
     SEQ_TRY(mix_mingru(m, ly, ws, s, st));
   } else if (ly.kind == UMB_MIX_ATTN_SSD) {
@@ -382,6 +411,8 @@ static int run_mixer(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWo
     SEQ_TRY(mix_attn_mlstm(m, ly, ws, s, st));
   } else if (ly.kind == UMB_MIX_DIFF_ATTN) {
     SEQ_TRY(mix_diff_attn(m, ly, ws, s, st));
+  } else if (ly.kind == UMB_MIX_SOFTMAX) {
+    SEQ_TRY(mix_softmax(m, ly, ws, s, st));
   } else if (ly.kind == UMB_MIX_ATTN_DELTA) {
     if (m->block == UMB_BLOCK_PARALLEL || m->streams >= 1 || m->groups != 1 || !ws->y2) return UMB_EINVAL;      // its seam is a single stream's
     SEQ_TRY(mix_attn_delta(m, ly, ws, s, st));
@@ -389,6 +420,16 @@ static int run_mixer(const UmbSeqModel* m, const UmbSeqLayer& ly, const UmbSeqWo
     return UMB_EINVAL;
   }
   return UMB_OK;
+}
+
+// logits of the R normed rows in ws->h, times logit_scale, then capped
+static int head_product(const UmbSeqModel* m, const UmbSeqWork* ws, const UmbSeqStep* s, hipStream_t st) {
+  const bool scaled = m->logit_scale != 0.f && m->logit_scale != 1.f;
+  if (m->logit_cap > 0.f)
+    return scaled ? UMB_EINVAL                                // no design has both
+                  : umb_seq_linear_cap(ws->logits, ws->h, m->head.w, m->head.bias, s->R, m->head.N, m->head.K, m->logit_cap, m->dtype, st);
+  SEQ_TRY(lin(m->head, ws->logits, ws->h, s->R, 0, m->dtype, st));
+  return scaled ? umb_seq_scale(ws->logits, (long)s->R * m->V, m->logit_scale, st) : UMB_OK;
 }
 
 // Layers whose sublayers both read the same residual: x <- x + (mixer(norm1 x) + ff(norm2 x)); one seam launch per layer adds
@@ -427,8 +468,7 @@ static int forward_parallel_blocks(const UmbSeqModel* m, const UmbSeqWork* ws, c
   if (s->R > 0) {
     // the final norm of the wanted rows only (a single stream read through the offset norm), then the head
     SEQ_TRY(umb_hc_read(nullptr, ws->h, ws->x, s->logit_rows, nullptr, m->final_norm, m->norm_offset, s->R, W, 1, m->eps, dt, st));
-    SEQ_TRY(lin(m->head, ws->logits, ws->h, s->R, 0, dt, st));
-    if (m->logit_scale != 0.f && m->logit_scale != 1.f) SEQ_TRY(umb_seq_scale(ws->logits, (long)s->R * m->V, m->logit_scale, st));
+    SEQ_TRY(head_product(m, ws, s, st));
   }
   return UMB_OK;
 }
@@ -499,7 +539,7 @@ extern "C" int umb_seq_forward(const UmbSeqModel* m, const UmbSeqWork* ws, const
       SEQ_TRY(umb_hc_read(nullptr, ws->h, ws->x, s->logit_rows, nullptr, m->final_norm, m->norm_offset, s->R, W, S, eps, dt, st));
     else
       SEQ_TRY(umb_seq_group_norm(nullptr, ws->h, ws->x, s->logit_rows, m->final_norm, s->R, W, groups, eps, dt, st));
-    SEQ_TRY(lin(m->head, ws->logits, ws->h, s->R, 0, dt, st));
+    SEQ_TRY(head_product(m, ws, s, st));
   }
   return UMB_OK;
 }

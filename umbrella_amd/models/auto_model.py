@@ -15,6 +15,7 @@ from .config import KNOWN, read_architecture
 from .fidizen import Fidizen
 from .gitopel import Gitopel
 from .llama import Llama
+from .potosun import Potosun
 from .tomopel import Tomopel
 from .tutunex import Tutunex
 from .zusuvik import Zusuvik
@@ -24,7 +25,7 @@ class AutoModelLM:
     # a local directory is resolved by the architecture its config.json names; directories that name none of these are
     # Hugging Face Llama / Qwen2 / Mistral checkpoints
     _ARCHITECTURE_MAPPING = {"Gitopel": Gitopel, "Fidizen": Fidizen, "Tomopel": Tomopel, "Zusuvik": Zusuvik,
-                             "Tutunex": Tutunex}
+                             "Tutunex": Tutunex, "Potosun": Potosun}
     _MODEL_MAPPING = {name: Llama for name in KNOWN}
     _OFFLOAD_MODEL_MAPPING = dict(_MODEL_MAPPING)
     _CUDAGRAPH_MODEL_MAPPING = dict(_MODEL_MAPPING)

@@ -223,11 +223,12 @@ class GLACfg:
 
 @dataclass
 class LatentAttnCfg:
-    """Softmax attention through low-rank latents: queries via a normed latent of ``q_rank``, keys / values via a normed
-    latent of ``kv_rank`` (the only thing cached, with one rotated key part of ``rot_dim`` shared by the heads); per head
-    ``dim`` unrotated + ``rot_dim`` rotated query / key features and ``vdim`` value features; interleaved rotary on the
-    first ``rot_dims`` of the rotated part; sliding window (0: none); a sink per head in the softmax denominator; a
-    sigmoid output gate."""
+    """Softmax attention through low-rank latents: queries via a normed latent of ``q_rank`` (0: straight from the input), keys /
+    values via a normed latent of ``kv_rank`` (the only thing cached, with one rotated key part of ``rot_dim`` shared by the
+    heads); per head ``dim`` unrotated + ``rot_dim`` rotated query / key features and ``vdim`` value features; rotary on the first
+    ``rot_dims`` of the rotated part (``rot_layout`` / ``rot_scaling`` other than the defaults: with ``q_rank`` 0 only); sliding
+    window (0: none); a sink per head in the softmax denominator; a sigmoid output gate, one per value feature or (``gate``
+    "head") one per head."""
     heads: int
     dim: int
     rot_dim: int
@@ -238,6 +239,9 @@ class LatentAttnCfg:
     rot_dims: int
     rot_base: float
     scale: float
+    rot_layout: str = "interleaved"
+    rot_scaling: Optional[dict] = None
+    gate: str = "element"
     kind: str = "latent_attention"
 
 
@@ -396,6 +400,57 @@ class DiffAttnCfg:
     kind: str = "diff_attention"
 
 
+def distance_buckets(rows: int, far: float, n: int) -> torch.Tensor:
+    """bucket of every distance 0 .. n - 1 (int64): the distance itself below rows // 2, then logarithmic steps that reach
+    the last row at distance ``far``; fp32 arithmetic"""
+    d = torch.arange(n, dtype=torch.int64)
+    half = rows // 2
+    if half < 1 or not far > half:
+        return torch.where(d < half, d, torch.full_like(d, rows - 1))
+    steps = torch.log(d.clamp_min(1).to(torch.float32) / half) / math.log(far / half) * (rows - half)
+    large = (half + steps.floor().to(torch.int64)).clamp(max=rows - 1)
+    return torch.where(d < half, d, large)
+
+
+def bias_by_distance(rel: torch.Tensor, far: float, max_len: int) -> torch.Tensor:
+    """the learned table [rows, heads] -> fp32 [heads, n_dist] indexed by the distance itself; distances from n_dist - 1 on
+    share the last entry (every distance the table tells apart, or every distance a sequence of max_len can hold)"""
+    rows = rel.shape[0]
+    n = int(max(1, min(max_len, max(math.ceil(far), rows // 2) + 1)))
+    b = distance_buckets(rows, far, n)
+    last = int((b == rows - 1).nonzero()[0]) if bool((b == rows - 1).any()) else n - 1
+    return rel.to(torch.float32)[b[:last + 1].to(rel.device)].t().contiguous()
+
+
+@dataclass
+class SoftmaxAttnCfg:
+    """Causal softmax attention with grouped query heads, each of its parts by choice: RMS-normed q and k per head (``qk_norm``, one
+    weight for all heads); rotary positions on the first ``rot_dims`` features (0: none); a learned bias per (distance bucket,
+    head) (``bias_far`` > 0; exact buckets below half the table, logarithmic up to ``bias_far``); keys of a sliding ``window`` (0:
+    none) or of the query's own run of ``chunk`` positions (0: none), the first ``keep_first`` tokens in any case; a learned score
+    per head in the softmax denominator (``sink``); one sigmoid gate per output feature (``gate``); ``v_mix``: values are mixed
+    with those of the model's first such layer before they are cached."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int = 0
+    keep_first: int = 0
+    chunk: int = 0
+    qk_norm: bool = False
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    rot_scaling: Optional[dict] = None
+    rot_layout: str = "half"
+    bias_far: float = 0.0
+    bias_rows: int = 0               # rows of the bias table: read from the tensor's shape at load
+    sink: bool = False
+    gate: bool = False
+    v_mix: bool = False
+    kind: str = "softmax_attention"
+
+
 @dataclass
 class AttnDeltaCfg:
     """Two mixers side by side that read the same input, each with its own output projection; ``pair_coef`` times the sum of the
@@ -430,7 +485,8 @@ class SeqLayerCfg:
     expert_ff: int = 0
     shared_ff: int = 0               # 0: no shared expert
     weights_of: int | None = None    # the layer uses that layer's tensors (with a cache and state of its own)
-    act: str = "silu_gated"          # "silu_gated": silu(W_gate h) * W_up h; "relu2": relu(W_up h)^2 (no gate) -- dense, experts, shared
+    act: str = "silu_gated"          # "silu_gated": silu(W_gate h) * W_up h; "relu2": relu(W_up h)^2 (no gate) -- dense, experts, shared;
+                                     # "gelu_gated": gelu(W_gate h) * W_up h (tanh form)
     route: str = "sigmoid_in"        # "sigmoid_in": sigmoid scores weigh the expert's input; "softmax_out": softmax scores,
                                      # chosen with a correction added, renormalised over the chosen, weigh its output;
                                      # "top_logits": the largest logits, softmax over the chosen alone, weigh its output
@@ -467,6 +523,7 @@ class SeqMixCfg:
     norm_offset: float = 0.0         # norm weights are stored around it: the factor is offset + w (streams >= 1, parallel blocks)
     block: str = "sequential"        # "parallel": both sublayers of a layer read the same residual, x + (mixer(norm1 x) + ff(norm2 x))
     logit_scale: float = 1.0         # the logits are multiplied by it
+    logit_cap: float = 0.0           # > 0: the logits become cap tanh(logits / cap)
 
     @property
     def num_hidden_layers(self):

@@ -2,14 +2,17 @@
 
 A model is a LIST of layers, each a token mixer -- windowed attention with pooled blocks, gated linear attention, latent
 attention, a minimal gated recurrence, softmax attention beside a state-space layer, retention, convolved softmax attention
-beside a matrix memory, differential attention (over its own or another layer's keys and values), or attention with a sink
-beside a gated delta rule -- plus an optional feed-forward (gated SiLU, PolyNorm, or routed experts with a shared one).  A sublayer reads either a grouped RMS norm of the residual stream or the
+beside a matrix memory, differential attention (over its own or another layer's keys and values), attention with a sink
+beside a gated delta rule, or softmax attention by form (window with kept first tokens or chunks, bias by distance, rotary, sink,
+gate, values mixed with an earlier layer's) -- plus an optional feed-forward (gated SiLU or gelu, PolyNorm, or routed experts with
+a shared one).  A sublayer reads either a grouped RMS norm of the residual stream or the
 stream itself through a short causal convolution; its output is normed before it is added back; or (``streams >= 1``) the
-residual is several streams that every sublayer reads as one combination and writes back to all.  A layer may use another
+residual is one or several streams that every sublayer reads as one combination and writes back to all (one stream without
+tables: the plain pre-norm residual).  A layer may use another
 layer's tensors with a cache and state of its own; or (``block == "parallel"``) both sublayers of a layer read the same
 residual and their outputs are added to it together.  The list, every size and every
 constant come from a ``SeqMixCfg`` (models/config.py); a design contributes a subclass that names its checkpoint tensors
-(models/gitopel.py, fidizen.py, tomopel.py, zusuvik.py, tutunex.py).
+(models/gitopel.py, fidizen.py, tomopel.py, zusuvik.py, tutunex.py, potosun.py).
 
 Unlike the tree-decoding ``Llama`` runtime this one serves MANY sequences: a step is a ragged batch (the rows of each
 sequence contiguous, nothing padded), key/value pages and recurrent-state slots are handed out by
@@ -32,9 +35,9 @@ from .base import LLMBase
 from .config import SeqMixCfg, rotary_frequencies, rotary_table
 
 KIND_CODE = {"attention": 0, "gla": 1, "latent_attention": 2, "mingru": 3, "attention_ssd": 4, "retention": 5,
-             "attention_mlstm": 6, "diff_attention": 7, "attention_delta": 8}
+             "attention_mlstm": 6, "diff_attention": 7, "attention_delta": 8, "softmax_attention": 9}
 FF_CODE = {"gated": 0, "polynorm": 1, "moe": 2}
-ACT_CODE = {"silu_gated": 0, "relu2": 1, "clamp_glu": 2}
+ACT_CODE = {"silu_gated": 0, "relu2": 1, "clamp_glu": 2, "gelu_gated": 3}
 ROUTE_CODE = {"sigmoid_in": 0, "softmax_out": 1, "top_logits": 2}
 BLOCK_CODE = {"sequential": 0, "parallel": 1}
 ROT_LAYOUT_CODE = {"half": 0, "interleaved": 1}
@@ -113,6 +116,7 @@ class SeqMixLM(LLMBase):
         assert tuple(self._top["embed"].shape) == (c.vocab_size, c.width), tuple(self._top["embed"].shape)
         L = len(c.layers)
         self._tensors, kv_layers, state_layers, latent_layers, n_conv, mixer_convs = [], [], [], [], 0, []
+        v_source = None                                 # (index, kv_heads, vdim) of the first layer that mixes values
         for i, ly in enumerate(c.layers):
             if ly.weights_of is not None:
                 # the tensors of another layer (which must own its tensors), a cache and state of this layer's own
@@ -131,6 +135,8 @@ class SeqMixLM(LLMBase):
                 t["cache_index"] = len(kv_layers)
                 kv_layers.append((m.kv_heads, m.dim, m.pool))
             elif m.kind == "latent_attention":
+                if m.q_rank and (m.rot_layout != "interleaved" or m.rot_scaling):
+                    raise ValueError("queries through a latent turn interleaved pairs by unscaled frequencies")
                 t["cache_index"] = len(latent_layers)
                 latent_layers.append(m.kv_rank + m.rot_dim)
             elif m.kind == "mingru":
@@ -170,6 +176,16 @@ class SeqMixLM(LLMBase):
                     if (src.kv_heads, src.dim, src.vdim) != (m.kv_heads, m.dim, m.vdim):
                         raise ValueError(f"layer {i}: kv_from wants equal key / value heads and sizes")
                     t["cache_index"] = self._tensors[m.kv_from]["cache_index"]
+            elif m.kind == "softmax_attention":
+                if m.heads % m.kv_heads:
+                    raise ValueError("heads must be a multiple of kv_heads")
+                t["cache_index"] = len(kv_layers)
+                kv_layers.append((m.kv_heads, m.dim, 0, m.vdim))
+                if m.v_mix and v_source is None:
+                    v_source = (i, m.kv_heads, m.vdim)
+                elif m.v_mix and (m.kv_heads, m.vdim) != v_source[1:]:
+                    raise ValueError(f"layer {i}: values mix with those of layer {v_source[0]}: equal key / value heads and value sizes")
+                t["v_mix"] = 0 if not m.v_mix else (1 if v_source[0] == i else 2)
             elif m.kind == "attention_delta":
                 if m.heads % m.kv_heads or m.s_heads % m.s_groups:
                     raise ValueError("heads must be a multiple of kv_heads on both sides")
@@ -184,12 +200,15 @@ class SeqMixLM(LLMBase):
             else:
                 t["cache_index"] = len(state_layers)
                 state_layers.append((m.heads, m.dim, m.vdim))
+            if m.kind == "latent_attention" and m.q_rank == 0:
+                freq, t["rot_mult"] = rotary_table(m.rot_base, m.rot_dims, m.rot_scaling) if m.rot_dims else (None, 1.0)
+                t["rot_freq"] = freq.to(dev) if freq is not None else None
             if m.kind in ("attention", "latent_attention") and "rot_freq" not in t:
                 i2 = torch.arange(m.rot_dims // 2, dtype=torch.float32)
                 t["rot_freq"] = (m.rot_base ** (-2 * i2 / m.rot_dims)).to(dev) if m.rot_dims else None     # fp32 frequencies
             if m.kind in ("retention", "attention_mlstm") and "rot_freq" not in t:
                 t["rot_freq"] = rotary_frequencies(m.rot_base, m.rot_dims, m.rot_scaling).to(dev) if m.rot_dims else None
-            if m.kind == "diff_attention":
+            if m.kind in ("diff_attention", "softmax_attention"):
                 freq, t["rot_mult"] = rotary_table(m.rot_base, m.rot_dims, m.rot_scaling) if m.rot_dims else (None, 1.0)
                 t["rot_freq"] = freq.to(dev) if freq is not None else None
             if c.canon_taps > 0:
@@ -199,6 +218,7 @@ class SeqMixLM(LLMBase):
         self.kv_cache = PagedSeqCache(kv_layers, state_layers, self.max_tokens, self.batch_size, dev, dt, page=self.page_size,
                                       latent_layers=latent_layers, conv_states=n_conv, conv_taps=c.canon_taps, width=c.width,
                                       mixer_convs=mixer_convs)
+        self._v_width = v_source[1] * v_source[2] if v_source else 0
         self._layer_structs = (UmbSeqLayer * L)()
         for i, (ly, t) in enumerate(zip(c.layers, self._tensors)):
             s, m = self._layer_structs[i], ly.mixer
@@ -223,8 +243,11 @@ class SeqMixLM(LLMBase):
                 s.q_rank, s.kv_rank, s.rot_dim, s.rot_dims, s.scale = m.q_rank, m.kv_rank, m.rot_dim, m.rot_dims, m.scale
                 s.window = m.window if m.window > 0 else 2 ** 30            # no window: every earlier position is seen
                 s.rot_freq = t["rot_freq"].data_ptr() if t["rot_freq"] is not None else None
-                s.uq, s.uk_t, s.uv = _linear(t["uq_w"]), t["uk_t"].data_ptr(), t["uv_w"].data_ptr()
-                s.dq_norm, s.dkv_norm = t["dq_norm"].data_ptr(), t["dkv_norm"].data_ptr()
+                s.rot_layout, s.rot_mult = ROT_LAYOUT_CODE[m.rot_layout], float(t.get("rot_mult", 1.0))
+                s.gate_head = int(m.gate == "head")
+                s.uk_t, s.uv, s.dkv_norm = t["uk_t"].data_ptr(), t["uv_w"].data_ptr(), t["dkv_norm"].data_ptr()
+                if m.q_rank:
+                    s.uq, s.dq_norm = _linear(t["uq_w"]), t["dq_norm"].data_ptr()
                 s.sink = t["sink"].data_ptr() if t.get("sink") is not None else None
                 s.kv = self.kv_cache.latent_struct(t["cache_index"])
             elif m.kind == "mingru":
@@ -272,6 +295,18 @@ class SeqMixLM(LLMBase):
                 s.rot_freq = t["rot_freq"].data_ptr() if t["rot_freq"] is not None else None
                 s.kv_shared, s.diff_lambda, s.out_mult = int(m.kv_from is not None), float(t["diff_lambda"]), 1.0 - float(m.diff)
                 s.kv = self.kv_cache.struct(t["cache_index"])
+            elif m.kind == "softmax_attention":
+                s.kv_heads, s.scale, s.window = m.kv_heads, float(m.scale), (m.window if m.window > 0 else 2 ** 30)
+                s.keep_first, s.chunk, s.gate_elem = int(m.keep_first), int(m.chunk), int(m.gate)
+                s.q_norm = t["q_norm"].data_ptr() if t.get("q_norm") is not None else None
+                s.k_norm = t["k_norm"].data_ptr() if t.get("k_norm") is not None else None
+                s.rot_dims, s.rot_layout, s.rot_mult = m.rot_dims, ROT_LAYOUT_CODE[m.rot_layout], float(t["rot_mult"])
+                s.rot_freq = t["rot_freq"].data_ptr() if t["rot_freq"] is not None else None
+                if t.get("dist_bias") is not None:                 # fp32 [heads][n_dist], indexed by the clamped distance
+                    s.dist_bias, s.n_dist = t["dist_bias"].data_ptr(), t["dist_bias"].shape[1]
+                s.attn_sink = t["attn_sink"].data_ptr() if t.get("attn_sink") is not None else None
+                s.v_mix, s.v_lambda = t["v_mix"], float(t.get("v_lambda", 0.0))
+                s.kv = self.kv_cache.struct(t["cache_index"])
             elif m.kind == "attention_delta":
                 s.kv_heads, s.scale, s.window = m.kv_heads, float(m.scale), 2 ** 30
                 s.q_norm, s.k_norm, s.attn_sink = t["q_norm"].data_ptr(), t["k_norm"].data_ptr(), t["attn_sink"].data_ptr()
@@ -309,7 +344,7 @@ class SeqMixLM(LLMBase):
         mdl.dtype, mdl.L, mdl.W, mdl.V, mdl.groups, mdl.eps = _lib.seq_dtype_code(dt), L, c.width, c.vocab_size, c.norm_groups, c.norm_eps
         mdl.embed_scale, mdl.canon_taps = float(c.embed_scale), int(c.canon_taps)
         mdl.streams, mdl.resid_mult, mdl.norm_offset = int(c.streams), float(c.resid_mult), float(c.norm_offset)
-        mdl.block, mdl.logit_scale = BLOCK_CODE[c.block], float(c.logit_scale)
+        mdl.block, mdl.logit_scale, mdl.logit_cap = BLOCK_CODE[c.block], float(c.logit_scale), float(c.logit_cap)
         mdl.embed, mdl.final_norm, mdl.head = self._top["embed"].data_ptr(), self._top["final_norm"].data_ptr(), _linear(self._top["head"])
         mdl.layers = C.cast(self._layer_structs, C.POINTER(UmbSeqLayer))
         self.reserve(self.max_step_tokens or 256)
@@ -337,7 +372,7 @@ class SeqMixLM(LLMBase):
             if m.kind == "latent_attention":
                 # act: query latent, then the attended latents; o: queries; mix: unrotated queries, then the gated heads;
                 # aux: queries carried into the latent space
-                ask(act=max(m.q_rank, m.heads * m.kv_rank), o=m.heads * (m.dim + m.rot_dim), mix=m.heads * max(m.dim, m.vdim),
+                ask(act=max(m.q_rank, m.heads * m.kv_rank), o=m.heads * (m.dim + m.rot_dim) if m.q_rank else 1, mix=m.heads * max(m.dim, m.vdim),
                     aux=m.heads * (m.kv_rank + m.rot_dim))
             elif m.kind == "mingru":
                 ask(mix=m.dim, aux=3 * m.dim + m.dim // 16 + 1)     # aux: piece summaries and start states of long stretches
@@ -364,6 +399,9 @@ class SeqMixLM(LLMBase):
             elif m.kind == "diff_attention":
                 # aux: queries of both maps, and room for the partial results of split keys (16 a row and more for few rows)
                 ask(aux=2 * m.heads * m.dim + 32 * m.heads * (m.vdim + 2) // (16 if T > 64 else 1) + 4, mix=m.heads * m.vdim)
+            elif m.kind == "softmax_attention":
+                # aux: queries, and room for the partial results of split keys (16 a row and more for few rows)
+                ask(aux=m.heads * m.dim + 16 * m.heads * (m.vdim + 2) // (16 if T > 64 else 1) + 4, mix=m.heads * m.vdim)
             elif m.kind == "attention_delta":
                 # aux: queries | delta-rule q, k, v, step sizes, log decays | the chunk kernels' scratch; mix: the two mixers' rows
                 up = lambda n: (n + 15) // 16 * 16                                                        # noqa: E731
@@ -394,6 +432,9 @@ class SeqMixLM(LLMBase):
         if c.block == "parallel" or any(ly.mixer.kind == "attention_delta" for ly in c.layers):
             b["y2"] = torch.zeros(T, c.width, dtype=f32, device=dev)     # its output; the second output projection's
             ws.y2 = b["y2"].data_ptr()
+        if self._v_width:                               # values that later layers of the step mix in
+            b["v_first"] = torch.zeros(T, self._v_width, dtype=f32, device=dev)
+            ws.v_first = b["v_first"].data_ptr()
         if top:
             pairs = T * top
             tiles = (pairs + 15) // 16 + max(ly.experts for ly in c.layers)          # the smallest tile size the forward picks

@@ -20,12 +20,11 @@ mechanism lives there and in csrc/seq_*.hip with its constants as parameters.
 from __future__ import annotations
 
 import json
-import math
 import os
 
 import torch
 
-from .config import AttnSSDCfg, MinGRUCfg, SeqLayerCfg, SeqMixCfg
+from .config import AttnSSDCfg, MinGRUCfg, SeqLayerCfg, SeqMixCfg, bias_by_distance, distance_buckets  # noqa: F401
 from .seqmix import SeqMixLM
 
 ARCHITECTURE = "Tomopel"
@@ -73,28 +72,6 @@ def config_from_dict(c: dict, name: str = "tomopel") -> SeqMixCfg:
 def config_from_dir(path: str) -> SeqMixCfg:
     with open(os.path.join(path, "config.json")) as f:
         return config_from_dict(json.load(f), name=os.path.basename(os.path.normpath(path)))
-
-
-def distance_buckets(rows: int, far: float, n: int) -> torch.Tensor:
-    """bucket of every distance 0 .. n - 1 (int64): the distance itself below rows // 2, then logarithmic steps that reach
-    the last row at distance ``far``; fp32 arithmetic"""
-    d = torch.arange(n, dtype=torch.int64)
-    half = rows // 2
-    if half < 1 or not far > half:
-        return torch.where(d < half, d, torch.full_like(d, rows - 1))
-    steps = torch.log(d.clamp_min(1).to(torch.float32) / half) / math.log(far / half) * (rows - half)
-    large = (half + steps.floor().to(torch.int64)).clamp(max=rows - 1)
-    return torch.where(d < half, d, large)
-
-
-def bias_by_distance(rel: torch.Tensor, far: float, max_len: int) -> torch.Tensor:
-    """the learned table [rows, heads] -> fp32 [heads, n_dist] indexed by the distance itself; distances from n_dist - 1 on
-    share the last entry (every distance the table tells apart, or every distance a sequence of max_len can hold)"""
-    rows = rel.shape[0]
-    n = int(max(1, min(max_len, max(math.ceil(far), rows // 2) + 1)))
-    b = distance_buckets(rows, far, n)
-    last = int((b == rows - 1).nonzero()[0]) if bool((b == rows - 1).any()) else n - 1
-    return rel.to(torch.float32)[b[:last + 1].to(rel.device)].t().contiguous()
 
 
 def tensor_shapes(cfg: SeqMixCfg, bias_rows: int = 16) -> dict:
