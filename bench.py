@@ -772,20 +772,23 @@ def main():
     ap.add_argument("--phase-timeout", type=float, default=240.0, help="watchdog per pp / tp phase, seconds")
     ap.add_argument("--dry-run", action="store_true", help="launch plumbing only (gloo, no GPU work)")
     ap.add_argument("--seed", type=int, default=0)
-    ap.add_argument("--family", default=None, choices=[None, "gitopel", "fidizen", "tomopel", "zusuvik", "tutunex"],
+    ap.add_argument("--family", default=None, choices=[None, "gitopel", "fidizen", "tomopel", "zusuvik", "tutunex", "potosun"],
                     help="gitopel: prefill / decode throughput of the sequence-mixer family beside Llama at equal size; "
                          "fidizen: of the Fidizen design beside Gitopel's attention layers at equal size; "
                          "tomopel: of the Tomopel design beside Gitopel at equal size; "
                          "zusuvik: of the Zusuvik design beside Tomopel at equal size; "
-                         "tutunex: of the Tutunex design beside Tomopel's and Gitopel's layers at equal size "
+                         "tutunex: of the Tutunex design beside Tomopel's and Gitopel's layers at equal size; "
+                         "potosun: of the Potosun design beside Gitopel's and Fidizen's layers at equal size "
                          "(scripts/bench_seqmix.py; one GPU) instead of the headline workload")
     sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "scripts"))
     import bench_seqmix
     bench_seqmix.add_args(ap)
     args = ap.parse_args()
-    if args.family in ("gitopel", "fidizen", "tomopel", "zusuvik", "tutunex"):
+    if args.family in ("gitopel", "fidizen", "tomopel", "zusuvik", "tutunex", "potosun"):
         if args.prompt_len == 128:
             args.prompt_len = 2048
+        if args.family == "potosun":
+            return bench_seqmix.run_potosun(args)
         if args.family == "tutunex":
             return bench_seqmix.run_tutunex(args)
         if args.family == "zusuvik":

@@ -26,6 +26,12 @@ synthetic ids.
         Tomopel's (attention beside a state-space layer of the same state size, a dense gated feed-forward), its
         differential layers beside Gitopel's windowed attention (window = chunk), at equal width, head rows and layer count
 
+    python bench.py --family potosun [--sizes 1b,8b] ...
+        Potosun (biased attention over a window with kept first tokens, chunked sink attention, latent attention with direct
+        queries; gated tanh-gelu), whole and kind by kind beside the closest existing layers: its two grouped-query kinds beside
+        Gitopel's windowed attention (window = window / chunk), its latent layers beside Fidizen's (dense feed-forward), at equal
+        width, heads, head and latent sizes, feed-forward width and layer count
+
 or directly: python scripts/bench_seqmix.py.  One JSON line: per size, ms and tokens/s of
   prefill   one prompt of --prompt-len tokens in one step (Llama: its chunked prompt path)
   decode    one token per step behind that prompt, batch 1 (both) and batch --batch (Gitopel; the Llama runtime is batch 1)
@@ -96,6 +102,29 @@ TUT_SIZES = {
 }
 
 
+# Potosun: "b" layers are biased attention (window, `keep` first tokens), "c" layers chunked attention with a sink, both heads x dim
+# over kv_heads with values mixed; "l" layers latent attention (l_heads of dim + rot, values l_vdim, latent kv_rank)
+POT_SIZES = {
+    "1b": dict(width=2048, ff=8192, heads=32, kv_heads=8, dim=64, vdim=64, window=512, keep=64, bias_max=2048, chunk=1024, l_heads=16,
+               l_dim=64, l_rot=32, l_vdim=64, kv_rank=256, l_window=512, bias_rows=32, pattern="clbb", vocab=32000),
+    "8b": dict(width=4096, ff=14336, heads=32, kv_heads=8, dim=128, vdim=128, window=1024, keep=64, bias_max=2048, chunk=1024, l_heads=32,
+               l_dim=128, l_rot=64, l_vdim=128, kv_rank=512, l_window=1024, bias_rows=32, pattern="clb", vocab=32000),
+}
+
+
+def potosun_config(s):
+    gqa = {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": s["dim"], "vdim": s["vdim"], "scale": s["dim"] ** -0.5, "v_mix": True}
+    kinds = {"b": ("attention", dict(gqa, bias_max=s["bias_max"], mask={"size": s["window"], "keep_first": s["keep"]})),
+             "c": ("attention_2", dict(gqa, mask={"size": s["chunk"]}, rot={"base": 500000.0, "dims": s["dim"]})),
+             "l": ("latent_attention", {"heads": s["l_heads"], "dim": s["l_dim"], "rot_dim": s["l_rot"], "vdim": s["l_vdim"], "kv_rank": s["kv_rank"],
+                                        "mask": {"size": s["l_window"]}, "scale": (s["l_dim"] + s["l_rot"]) ** -0.5,
+                                        "rot": {"base": 10000.0, "dims": s["l_rot"],
+                                                "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}})}
+    layers = [{"type": kinds[ch][0], "mixer": kinds[ch][1], "mlp": {"kind": "dense", "ff": s["ff"]}} for ch in s["pattern"]]
+    return {"architecture": "Potosun", "layers": layers, "norm": {"eps": 1e-6}, "embedding": {"scale": s["width"] ** 0.5}, "logit_softcap": 30.0,
+            "vocab": s["vocab"], "width": s["width"]}
+
+
 def tutunex_config(s):
     layers, last = [], None
     for i, ch in enumerate(s["pattern"]):
@@ -164,7 +193,7 @@ def fidizen_config(s):
              "scale": (s["dim"] + s["rot"]) ** -0.5}
     layers = []
     for i in range(s["layers"]):
-        if i % 2 == 0:
+        if i % 2 == 0 or s.get("all_dense"):
             mlp = {"kind": "dense", "ff": s["ff"]}
         else:
             mlp = {"kind": "moe", "router": {"experts": s["experts"], "top": s["top"]}, "expert": {"ff": s["ff"] // 4},
@@ -200,7 +229,7 @@ def device_state(cfg, dtype, seed=0, rank=16, shapes=None, zero_norms=False):
             sd[name] = (base.cuda() + 0.05 * torch.randn(shape, generator=g, device="cuda")).to(dtype)
         elif "norm" in leaf:
             sd[name] = torch.full(shape, 0.0 if zero_norms and "mix." not in name else 1.0, dtype=dtype, device="cuda")
-        elif len(shape) == 1:
+        elif len(shape) <= 1:
             sd[name] = (0.1 * torch.randn(shape, generator=g, device="cuda")).to(dtype)
         else:
             sd[name] = (torch.randn(shape, generator=g, device="cuda", dtype=torch.float32) / shape[1] ** 0.5).to(dtype)
@@ -216,16 +245,20 @@ def timed(fn, reps):
     return (time.time() - t0) / reps * 1e3
 
 
-def bench_gitopel(s, args, dtype, fidizen=False, tomopel=False, zusuvik=False, tutunex=False):
+def bench_gitopel(s, args, dtype, fidizen=False, tomopel=False, zusuvik=False, tutunex=False, potosun=False):
     from umbrella_amd.models import fidizen as fid
     from umbrella_amd.models import gitopel
+    from umbrella_amd.models import potosun as pot
     from umbrella_amd.models import tomopel as tom
     from umbrella_amd.models import tutunex as tut
     from umbrella_amd.models import zusuvik as zus
     B, P, steps = args.batch, args.prompt_len, args.decode_steps
     kw = dict(batch_size=B + 1, max_length=P + 2 * steps + 8, max_tokens=(B + 1) * (P + 2 * steps + 8), device="cuda:0",
               dtype=dtype, max_step_tokens=max(P, B))
-    if tutunex:
+    if potosun:
+        cfg = pot.config_from_dict(potosun_config(s))
+        m = pot.Potosun("bench", state_dict=device_state(cfg, dtype, shapes=pot.tensor_shapes(cfg, s["bias_rows"])), config=cfg, **kw)
+    elif tutunex:
         cfg = tut.config_from_dict(tutunex_config(s))
         m = tut.Tutunex("bench", state_dict=device_state(cfg, dtype, shapes=tut.tensor_shapes(cfg)), config=cfg, **kw)
     elif zusuvik:
@@ -295,6 +328,37 @@ def bench_llama(s, args, dtype):
     out["decode_b1"] = {"context": P, "ms_per_step": round(ms, 4), "tokens_per_s": round(1 / ms * 1e3),
                         "weight_stream_TBs": round(m.weight_bytes() / ms / 1e9, 3)}
     return out
+
+
+def run_potosun(args):
+    """Potosun as a whole, then its kinds of layers two at a time beside the closest existing ones at equal size: biased and chunked
+    attention beside Gitopel's windowed attention, latent attention beside Fidizen's with a dense feed-forward"""
+    import __graft_entry__ as ge
+    ge.build_seq()
+    dtype = torch.bfloat16
+    res = {}
+    for name in args.sizes.split(","):
+        s = POT_SIZES[name]
+        r = res[name] = {"shape": dict(s)}
+        runs = [("potosun", dict(s), dict(potosun=True))]
+        if not args.no_gitopel:
+            g = dict(width=s["width"], ff=s["ff"], heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], pool=16, pattern="aa", vocab=s["vocab"])
+            f = dict(width=s["width"], ff=s["ff"], heads=s["l_heads"], dim=s["l_dim"], rot=s["l_rot"], vdim=s["l_vdim"], q_rank=FID_SIZES[name]["q_rank"],
+                     kv_rank=s["kv_rank"], window=s["l_window"], experts=8, top=2, layers=2, all_dense=True, vocab=s["vocab"])
+            runs += [("potosun_biased_layers", dict(s, pattern="bb"), dict(potosun=True)),
+                     ("gitopel_attention_layers_equal_window", dict(g, window=s["window"]), {}),
+                     ("potosun_chunked_layers", dict(s, pattern="cc"), dict(potosun=True)),
+                     ("gitopel_attention_layers_window_of_a_chunk", dict(g, window=s["chunk"]), {}),
+                     ("potosun_latent_layers", dict(s, pattern="ll"), dict(potosun=True)),
+                     ("fidizen_dense_layers_equal_size", f, dict(fidizen=True))]
+        for key, shape, kind in runs:
+            r[key] = bench_gitopel(shape, args, dtype, **kind)
+            torch.cuda.empty_cache()
+    line = {"metric": "prefill / decode throughput, Potosun whole and kind by kind beside the closest layers at equal size",
+            "unit": "tokens/s", "dtype": "bf16", "data": "synthetic: random weights, random ids", "n_gpus": 1,
+            "prompt_len": args.prompt_len, "decode_steps": args.decode_steps, "batch": args.batch, "sizes": res}
+    print(json.dumps(line), flush=True)
+    return line
 
 
 def run_fidizen(args):
@@ -438,7 +502,7 @@ def add_args(ap):
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--prompt-len", type=int, default=2048)
-    ap.add_argument("--family", default="gitopel", choices=["gitopel", "fidizen", "tomopel", "zusuvik", "tutunex"])
+    ap.add_argument("--family", default="gitopel", choices=["gitopel", "fidizen", "tomopel", "zusuvik", "tutunex", "potosun"])
     add_args(ap)
     a = ap.parse_args()
-    {"fidizen": run_fidizen, "tomopel": run_tomopel, "zusuvik": run_zusuvik, "tutunex": run_tutunex}.get(a.family, run)(a)
+    {"fidizen": run_fidizen, "tomopel": run_tomopel, "zusuvik": run_zusuvik, "tutunex": run_tutunex, "potosun": run_potosun}.get(a.family, run)(a)
