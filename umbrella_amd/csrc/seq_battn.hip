@@ -536,7 +536,12 @@ __global__ __launch_bounds__(256) void bsa_attend_mfma_kernel(u16* __restrict__ 
   u16* k_s = bsa_lds;                                 // [32][LD]
   u16* v_t = bsa_lds + 32 * LD;                       // [E][LT]
   const int b = blockIdx.y;
-  const int n = seq_len[b], q0 = blockIdx.x * 16;
+  // How many keys a tile sees depends on its place in the chunk (or, without a window, in the sequence).  Workgroups that share a CU
+  // are about 256 apart in launch order, which is the same tile of another head block: every other run of 256 takes the tiles from the
+  // far end, so a CU's workgroups add up to about the same work.
+  const int row = b + (int)gridDim.y * (int)blockIdx.z, run = gridDim.x < 256 ? 256 / gridDim.x : 1;
+  const int tile = (row / run) & 1 ? (int)(gridDim.x - 1 - blockIdx.x) : (int)blockIdx.x;
+  const int n = seq_len[b], q0 = tile * 16;
   if (q0 >= n) return;                                // the whole workgroup
   const int hpg = H / G, hblocks = (hpg + 4 * HW - 1) / (4 * HW);
   const int g = blockIdx.z / hblocks;
@@ -803,6 +808,7 @@ extern "C" int umb_attn_attend_tiled(void* out, int ldo, const float* q, const U
   } while (0)
 #define BSA_MFMA_SHAPE()                                                                                                   \
   if (maps == 2) { if (D <= 128 && E <= 128) BSA_MFMA(4, 8, 2, 2); else BSA_MFMA(8, 16, 2, 2); }                           \
+  else if (D <= 64 && E <= 64) { if (hpg > 4) BSA_MFMA(2, 4, 2, 1); else BSA_MFMA(2, 4, 1, 1); }                           \
   else if (D <= 128 && E <= 128) { if (hpg > 4) BSA_MFMA(4, 8, 2, 1); else BSA_MFMA(4, 8, 1, 1); }                         \
   else BSA_MFMA(8, 16, 1, 1)
   if (dtype == UMB_SEQ_BF16) { using P = BF16; BSA_MFMA_SHAPE(); }

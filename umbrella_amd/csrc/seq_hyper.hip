@@ -62,7 +62,26 @@ __global__ __launch_bounds__(256) void hc_seam_kernel(float* __restrict__ x, typ
     }
     return u;
   };
-  if constexpr (EPT > 0) {
+  float wn[NE];                                          // the next norm's weights, fetched with the row
+  if constexpr (EPT > 0 && NS == 1) {
+    // one stream: the whole row is in flight before the first element is written
+    float xo[NE], yo[NE];
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e, ic = i < W ? i : W - 1;
+      xo[e] = xr[ic];
+      yo[e] = yr[ic];
+      wn[e] = read ? ldf<P>(w_next + ic) : 0.f;
+    }
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e;
+      const float a = tb.mix[0][0] * xo[e] + tb.out[0] * (m * yo[e]);
+      if (i < W) xr[i] = a;
+      uv[e] = i < W ? tb.in[0] * a : 0.f;
+      ss += uv[e] * uv[e];
+    }
+  } else if constexpr (EPT > 0) {
 #pragma unroll
     for (int e = 0; e < EPT; ++e) {
       const int i = threadIdx.x + 256 * e;
@@ -79,7 +98,7 @@ __global__ __launch_bounds__(256) void hc_seam_kernel(float* __restrict__ x, typ
 #pragma unroll
     for (int e = 0; e < EPT; ++e) {
       const int i = threadIdx.x + 256 * e;
-      if (i < W) stf<P>(h + (long)t * W + i, uv[e] * f * (offset + ldf<P>(w_next + i)));
+      if (i < W) stf<P>(h + (long)t * W + i, uv[e] * f * (offset + (NS == 1 ? wn[e] : ldf<P>(w_next + i))));
     }
   } else {
     for (int i = threadIdx.x; i < W; i += 256) {
@@ -92,7 +111,8 @@ __global__ __launch_bounds__(256) void hc_seam_kernel(float* __restrict__ x, typ
 }
 
 // read alone (rows gathered): u = sum_s in[s] x_s -> u_out (fp32) and / or h = norm(u) * (offset + w)
-template <typename P>
+// (EPT > 0: one stream, the row stays in registers between the two passes)
+template <typename P, int EPT>
 __global__ __launch_bounds__(256) void hc_read_kernel(float* __restrict__ u_out, typename El<P>::type* __restrict__ h,
                                                       const float* __restrict__ x, const int* __restrict__ rows,
                                                       const float* __restrict__ in, const typename El<P>::type* __restrict__ w,
@@ -106,6 +126,32 @@ __global__ __launch_bounds__(256) void hc_read_kernel(float* __restrict__ u_out,
     for (int s = 0; s < S; ++s) u += (in ? in[s] : 1.f) * xr[(long)s * W + i];
     return u;
   };
+  if constexpr (EPT > 0) {
+    const float in0 = in ? in[0] : 1.f;
+    float uv[EPT], wv[EPT];
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e, ic = i < W ? i : W - 1;
+      uv[e] = xr[ic];
+      wv[e] = h ? ldf<P>(w + ic) : 0.f;
+    }
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e;
+      uv[e] = i < W ? in0 * uv[e] : 0.f;
+      if (u_out && i < W) u_out[(long)t * W + i] = uv[e];
+      ss += uv[e] * uv[e];
+    }
+    if (!h) return;
+    ss = block_sum<256>(ss, red);
+    const float f = 1.f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = threadIdx.x + 256 * e;
+      if (i < W) stf<P>(h + (long)t * W + i, uv[e] * f * (offset + wv[e]));
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < W; i += 256) {
     const float u = comb(i);
     if (u_out) u_out[(long)t * W + i] = u;
@@ -119,7 +165,7 @@ __global__ __launch_bounds__(256) void hc_read_kernel(float* __restrict__ u_out,
 
 // every stream <- embed[token] * scale; h <- the first read.  With all streams equal u = (sum_s in[s]) e, formed as the
 // same sum the read kernel forms, so a one-token step and a prompt give the same bits.
-template <typename P>
+template <typename P, int EPT>
 __global__ __launch_bounds__(256) void hc_embed_kernel(float* __restrict__ x, typename El<P>::type* __restrict__ h,
                                                        const typename El<P>::type* __restrict__ embed,
                                                        const int* __restrict__ tokens, float scale, const float* __restrict__ in,
@@ -137,6 +183,33 @@ __global__ __launch_bounds__(256) void hc_embed_kernel(float* __restrict__ x, ty
     for (int s = 0; s < S; ++s) u += (in ? in[s] : 1.f) * e;
     return u;
   };
+  if constexpr (EPT > 0) {                               // one stream
+    const float in0 = in ? in[0] : 1.f;
+    float ev[EPT], wv[EPT];
+#pragma unroll
+    for (int k = 0; k < EPT; ++k) {
+      const int i = threadIdx.x + 256 * k, ic = i < W ? i : W - 1;
+      ev[k] = ldf<P>(er + ic);
+      wv[k] = h ? ldf<P>(w + ic) : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < EPT; ++k) {
+      const int i = threadIdx.x + 256 * k;
+      const float e = ev[k] * scale;
+      if (i < W) xr[i] = e;
+      ev[k] = i < W ? in0 * e : 0.f;
+      ss += ev[k] * ev[k];
+    }
+    if (!h) return;
+    ss = block_sum<256>(ss, red);
+    const float f = 1.f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+    for (int k = 0; k < EPT; ++k) {
+      const int i = threadIdx.x + 256 * k;
+      if (i < W) stf<P>(h + (long)t * W + i, ev[k] * f * (offset + wv[k]));
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < W; i += 256) {
     const float e = ldf<P>(er + i) * scale;
     for (int s = 0; s < S; ++s) xr[(long)s * W + i] = e;
@@ -152,11 +225,17 @@ __global__ __launch_bounds__(256) void hc_embed_kernel(float* __restrict__ x, ty
 extern "C" int umb_hc_embed(float* x, void* h, const void* embed, const int* tokens, float scale, const float* in, const void* w,
                             float offset, int T, int W, int V, int S, float eps, int dtype, hipStream_t st) {
   if (T < 1 || W < 1 || V < 1 || S < 1 || S > HC_MAXS || !x || !embed || !tokens || (h && !w)) return UMB_EINVAL;
+#define HC_EMBED(EPT)                                                                                                           \
+  hipLaunchKernelGGL((hc_embed_kernel<P, EPT>), dim3(T), dim3(256), 0, st, x, (E*)h, (const E*)embed, tokens, scale, in, (const E*)w, \
+                     offset, W, V, S, eps)
   DISPATCH_SEQ_DTYPE(dtype, {
     typedef typename El<P>::type E;
-    hipLaunchKernelGGL(hc_embed_kernel<P>, dim3(T), dim3(256), 0, st, x, (E*)h, (const E*)embed, tokens, scale, in, (const E*)w,
-                       offset, W, V, S, eps);
+    if (S > 1 || W > 4096) HC_EMBED(0);
+    else if (W <= 1024) HC_EMBED(4);
+    else if (W <= 2048) HC_EMBED(8);
+    else HC_EMBED(16);
   })
+#undef HC_EMBED
   UMB_LAUNCH_CHECK();
   return UMB_OK;
 }
@@ -193,10 +272,16 @@ extern "C" int umb_hc_seam(float* x, void* h, const float* y, const float* mix, 
 extern "C" int umb_hc_read(float* u_out, void* h, const float* x, const int* rows, const float* in, const void* w, float offset,
                            int R, int W, int S, float eps, int dtype, hipStream_t st) {
   if (R < 1 || W < 1 || S < 1 || S > HC_MAXS || !x || (!u_out && !h) || (h && !w)) return UMB_EINVAL;
+#define HC_READ(EPT)                                                                                                            \
+  hipLaunchKernelGGL((hc_read_kernel<P, EPT>), dim3(R), dim3(256), 0, st, u_out, (E*)h, x, rows, in, (const E*)w, offset, W, S, eps)
   DISPATCH_SEQ_DTYPE(dtype, {
     typedef typename El<P>::type E;
-    hipLaunchKernelGGL(hc_read_kernel<P>, dim3(R), dim3(256), 0, st, u_out, (E*)h, x, rows, in, (const E*)w, offset, W, S, eps);
+    if (S > 1 || W > 4096) HC_READ(0);
+    else if (W <= 1024) HC_READ(4);
+    else if (W <= 2048) HC_READ(8);
+    else HC_READ(16);
   })
+#undef HC_READ
   UMB_LAUNCH_CHECK();
   return UMB_OK;
 }

@@ -64,8 +64,9 @@ static inline bool epi_dual(int epi) { return epi == EPI_SILU_MUL || epi == EPI_
 static inline bool epi_plain(int epi) {
   return epi == EPI_F32 || epi == EPI_DT || epi == EPI_SILU_MUL || epi == EPI_RELU2 || epi == EPI_GELU_MUL;
 }
-// 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))
-__device__ __forceinline__ float gelu_tanhf_(float z) { return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
+// 0.5 z (1 + tanh(u)) with u = sqrt(2 / pi) (z + 0.044715 z^3), as z / (1 + e^(-2 u)): the same function, one exponential, and no
+// cancellation where tanh is near -1
+__device__ __forceinline__ float gelu_tanhf_(float z) { return z / (1.f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z))); }
 __device__ __forceinline__ float glu_pair(int epi, float g, float u, float limit, float alpha) {
   if (epi == EPI_CLAMP_GLU) {
     g = fminf(g, limit);
