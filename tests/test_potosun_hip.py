@@ -208,7 +208,8 @@ def _case(kind, seed, W=24, rows=8, **kw):
 
 BIASED = [((4, 2, 8, 12), (9, 3, 14), 8, [19]), ((3, 1, 7, 5), (1, 0, 9), 6, [1] * 12), ((3, 1, 7, 5), (5, 1, 30), 16, [2, 9, 1, 1, 17, 3]),
           ((2, 2, 16, 16), (8, 11, 20), 8, [40, 1, 1, 30, 2, 2]), ((10, 2, 40, 80), (33, 16, 60), 12, [70, 1, 64, 3, 62]),
-          ((8, 1, 72, 144), (50, 6, 45), 32, [33, 20, 1, 48]), ((2, 1, 136, 272), (12, 2, 90), 8, [17, 2, 16]), ((4, 4, 24, 48), (20, 70, 25), 4, [64, 1, 1, 31])]
+          ((8, 1, 72, 144), (50, 6, 45), 32, [33, 20, 1, 48]), ((2, 1, 136, 272), (12, 2, 90), 8, [17, 2, 16]), ((4, 4, 24, 48), (20, 70, 25), 4, [64, 1, 1, 31]),
+          ((12, 2, 56, 64), (21, 5, 40), 8, [50, 1, 2, 17])]
 
 
 @BOTH
@@ -288,6 +289,33 @@ def test_edges_of_one_outstanding_key(lib, dtype, page, mask):
             like = (got.double().cpu().view(n, H, E) / torch.linspace(3.0, 8.0, E).double()).mean(-1).mean(-1)       # 1 where the mark was read
             outside = [i for i in range(n) if i not in inside]
             assert float(like[inside].min()) > 0.95 and (not outside or float(like[outside].abs().max()) < 0.5), (far, splits[:3])
+
+
+@pytest.mark.parametrize("mask", ["window", "chunk"])
+@pytest.mark.parametrize("n,H,G", [(330, 16, 16), (700, 24, 8)])
+def test_prompt_tiles_dealt_from_both_ends(lib, mask, n, H, G):
+    """enough head blocks that some of them walk the prompt's tiles from the far end: two sequences of unequal length in one launch"""
+    from oracle import potosun as O
+    from potosun_helpers import Steps, close, dev, rnd, zeros
+    D, E, size, keep, dtype = 16, 16, 45, 6, torch.bfloat16
+    counts = [n, 61]
+    T = sum(counts)
+    q, k, v = 2 * rnd((T, H, D), 1), rnd((T, G, D), 2), rnd((T, G, E), 3)
+    cache = _cache(G, D, E, dtype, 16)
+    slots = [cache.open("a"), cache.open("b")]
+    st = Steps(counts, [cache.extend("a", n), cache.extend("b", 61)], slots)
+    proj, qq, out = dev(torch.cat([q.reshape(T, -1), k.reshape(T, -1), v.reshape(T, -1)], dim=1)), zeros(T, H * D), zeros(T, H * E, dtype=dtype)
+    call("umb_attn_prep", qq, cache.struct(0), proj, proj.shape[1], 1, None, None, 0, 0, st.d["pos"], st.d["slot"], None, 0, 0, 1.0, T, H, G, D, E, 1, 0.0,
+         0, 1e-5, code(dtype))
+    f = form(0, None, keep) if mask == "window" else form(size)
+    _attend(lib, out, H * E, qq, cache.struct(0), st, H, G, D, E, size if mask == "window" else 2 ** 30, 0.4, f, dtype, False)
+    sees = (lambda i, j: O.sees_window(i, j, size, keep)) if mask == "window" else (lambda i, j: O.sees_chunk(i, j, size))
+    at = 0
+    for c in counts:
+        z = slice(at, at + c)
+        want = O.attend(q[z].double(), k[z].double(), v[z].double(), O.visible(torch.arange(c), c, sees), 0.4)
+        assert close(out[z], want.reshape(c, -1), BF16_TOL)
+        at += c
 
 
 @BOTH
