@@ -59,11 +59,14 @@ def rotate(x, pos, rot, interleaved: bool):
 
 
 def distance_bucket(n: int, rows: int, far: float) -> int:
-    """row of the bias table at distance n: the distance itself below rows // 2, then logarithmic steps, the last row from ``far`` on"""
+    """row of the bias table at distance n: the distance itself below rows // 2, then logarithmic steps, the last row from ``far`` on (a whole
+    number of steps counts as that number although the quotient of two rounded logarithms may fall short of it)"""
     half = rows // 2
     if n < half:
         return n
-    return min(rows - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (rows - half)))
+    steps = math.log(n / half) / math.log(far / half) * (rows - half)
+    whole = round(steps)
+    return min(rows - 1, half + (whole if abs(steps - whole) < 1e-9 else math.floor(steps)))
 
 
 # ------------------------------------------------------------------ which keys a position sees

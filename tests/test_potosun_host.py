@@ -54,7 +54,7 @@ def test_synthetic_checkpoint_names_and_shapes():
     assert "l4.norm2" not in sd and sd["l6.norm2"].shape == (40,) and sd["head"].shape == (90, 40)
 
 
-@pytest.mark.parametrize("rows,far", [(8, 14), (8, 30.0), (16, 128), (16, 100), (32, 2048), (2, 40), (12, 7), (4, 3)])
+@pytest.mark.parametrize("rows,far", [(8, 14), (8, 30.0), (16, 128), (16, 100), (32, 2048), (2, 40), (12, 7), (4, 3), (10, 160), (48, 81)])
 def test_bias_table_by_distance_equals_the_bucket_function(rows, far):
     from oracle import potosun as O
     from umbrella_amd.models.config import bias_by_distance
@@ -66,6 +66,16 @@ def test_bias_table_by_distance_equals_the_bucket_function(rows, far):
         assert float(tab[0, min(d, tab.shape[1] - 1)]) == want and float(tab[1, min(d, tab.shape[1] - 1)]) == want + 100
     short = bias_by_distance(rel, float(far), max_len=3)                   # a table for short sequences only
     assert short.shape[1] <= 3 and torch.equal(short, tab[:, :short.shape[1]])
+
+
+def test_distances_a_whole_number_of_steps_out():
+    """far / half = 2^5 over 5 steps, 1.5^3 over 24: the distance half 2^k (half 1.5^k) opens its bucket"""
+    from oracle import potosun as O
+    from umbrella_amd.models.config import distance_buckets
+    for rows, far, at in ((10, 160, {10: 6, 9: 5, 20: 7, 19: 6, 80: 9, 79: 8}), (48, 81, {36: 32, 35: 31, 54: 40, 53: 39})):
+        b = distance_buckets(rows, float(far), far + 2)
+        for n, want in at.items():
+            assert int(b[n]) == want and O.distance_bucket(n, rows, float(far)) == want, (rows, n)
 
 
 def test_rotation_tables_and_layouts():

@@ -402,13 +402,14 @@ class DiffAttnCfg:
 
 def distance_buckets(rows: int, far: float, n: int) -> torch.Tensor:
     """bucket of every distance 0 .. n - 1 (int64): the distance itself below rows // 2, then logarithmic steps that reach
-    the last row at distance ``far``; fp32 arithmetic"""
+    the last row at distance ``far``.  Float64, and a step count within 1e-9 of an integer is that integer: distances where the
+    logarithms' ratio is a whole number of steps stand on the upper side whatever way their quotient rounds"""
     d = torch.arange(n, dtype=torch.int64)
     half = rows // 2
     if half < 1 or not far > half:
         return torch.where(d < half, d, torch.full_like(d, rows - 1))
-    steps = torch.log(d.clamp_min(1).to(torch.float32) / half) / math.log(far / half) * (rows - half)
-    large = (half + steps.floor().to(torch.int64)).clamp(max=rows - 1)
+    steps = torch.log(d.clamp_min(1).to(torch.float64) / half) / math.log(far / half) * (rows - half)
+    large = (half + (steps + 1e-9).floor().to(torch.int64)).clamp(max=rows - 1)
     return torch.where(d < half, d, large)
 
 
